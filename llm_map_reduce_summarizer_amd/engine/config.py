@@ -105,6 +105,89 @@ class SSMSpec:
 
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """YaRN interpolation of rotary frequencies: pairs that turn fewer than ``slow`` times over ``original`` positions
+    are slowed down by ``factor``, those that turn more than ``fast`` times are kept, with a linear ramp between; cosine
+    and sine are multiplied by 0.1 ln(factor) + 1."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class RotarySpec:
+    """Rotate-half positions on ``dims`` dimensions: pair (i, i + dims / 2) turns by position * base^(-2 i / dims)."""
+    dims: int
+    base: float
+    scaling: Optional[YarnSpec] = None
+
+    def __post_init__(self):
+        if self.dims <= 0 or self.dims % 2:
+            raise ValueError("rotary positions need an even number of dimensions, got %d" % self.dims)
+
+
+@dataclass(frozen=True)
+class LatentSpec:
+    """Latent attention: keys and values of every head are expanded from one normed latent of ``kv_rank`` per token
+    (plus one rotated key part of ``rot.dims`` shared by the heads), queries from a normed latent of ``q_rank``.  Only
+    the latent and the rotated part are cached.  ``kv_from``: the layer whose cache this one reads instead of having
+    its own."""
+    heads: int
+    dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    rot: RotarySpec
+    scale: float
+    kv_from: Optional[int] = None
+
+    @property
+    def rot_dim(self) -> int:
+        return self.rot.dims
+
+
+@dataclass(frozen=True)
+class DeltaSpec:
+    """Gated delta rule: head h uses query / key head h // (heads // kv_heads); ``conv`` taps of the causal short
+    convolutions of q, k and v; one decay and one step size per head; head-wise output norm with a silu gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+    def __post_init__(self):
+        if self.kv_heads <= 0 or self.heads % self.kv_heads or self.conv < 1:
+            raise ValueError("delta mixer: heads %d / kv_heads %d / conv %d do not fit"
+                             % (self.heads, self.kv_heads, self.conv))
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        """Channels of the short convolutions: q, k and v."""
+        return 2 * self.kv_heads * self.dim + self.inner
+
+
+@dataclass(frozen=True)
+class GeluSpec:
+    """Plain feed-forward: W_down gelu(W_up h), the tanh form of gelu."""
+    ff: int
+
+
+@dataclass(frozen=True)
+class BigramSpec:
+    """A second embedding, indexed by the pair (previous token, token): row (previous * mul_prev + token * mul_cur)
+    mod ``buckets``, and row ``buckets`` for a sequence's first token."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass(frozen=True)
 class GLUSpec:
     """Clamped gated linear unit: g = min(g, limit), u = clamp(u, -limit, limit), y = g sigmoid(alpha g) (u + shift)."""
     ff: int
@@ -115,34 +198,54 @@ class GLUSpec:
 
 @dataclass(frozen=True)
 class LayerSpec:
-    """One pre-norm layer: attention and / or a state-space mixer side by side on the same normed input (summed
-    with their scales), then an optional feed-forward."""
+    """One pre-norm layer: the mixers given (attention beside a state-space mixer, or latent attention, or a delta rule)
+    on the same normed input, summed (attention and state-space mixer with their scales), and an optional feed-forward
+    -- after the mixers behind a norm of its own, or, ``parallel``, on the mixers' input and added with them."""
     attn: Optional[AttnSpec] = None
     ssm: Optional[SSMSpec] = None
-    mlp: Optional[GLUSpec] = None
+    mlp: Optional[Union[GLUSpec, GeluSpec]] = None
     attn_scale: float = 1.0
     ssm_scale: float = 1.0
+    latent: Optional[LatentSpec] = None
+    delta: Optional[DeltaSpec] = None
+    parallel: bool = False
 
     def __post_init__(self):
-        if self.attn is None and self.ssm is None:
+        if all(m is None for m in (self.attn, self.ssm, self.latent, self.delta)):
             raise ValueError("a layer needs a mixer")
+        if self.mlp is not None and isinstance(self.mlp, GeluSpec) != self.parallel:
+            raise ValueError("a parallel layer has a plain feed-forward, a sequential one a gated one")
 
 
 @dataclass(frozen=True)
 class HybridConfig:
-    """A decoder whose layers are listed one by one (engine/hybrid.py HybridModel): fp32 residual stream, sinusoidal
-    absolute positions added to the scaled embedding, RMS norms with weights stored around zero."""
+    """A decoder whose layers are listed one by one (engine/hybrid.py HybridModel): fp32 residual stream; the scaled
+    embedding plus sinusoidal absolute positions (``pos_base``), or plus a bigram embedding and an RMS norm
+    (``bigram``); the model's RMS norms multiply by (``norm_offset`` + weight)."""
     name: str
     vocab_size: int
     hidden: int
     layers: Tuple[LayerSpec, ...]
     rms_eps: float = 1e-6
     embed_scale: float = 1.0
-    pos_base: float = 10000.0
-    norm_offset: float = 1.0  # the model's norms multiply by (offset + w)
+    pos_base: Optional[float] = 10000.0
+    norm_offset: float = 1.0
     max_position: int = 131072
     init_std: float = 0.02
-    tp_shardable = False  # recurrent mixers and the whole-projection q / k norm are not sharded
+    bigram: Optional[BigramSpec] = None
+    tp_shardable = False  # recurrent mixers, whole-projection norms and shared latents are not sharded
+
+    def __post_init__(self):
+        for i, la in enumerate(self.layers):
+            s = la.latent
+            if s is None or s.kv_from is None:
+                continue
+            j = s.kv_from
+            o = self.layers[j].latent if 0 <= j < i else None
+            if o is None or o.kv_from is not None:
+                raise ValueError("layer %d takes its latents from layer %r, which has none of its own before it" % (i, j))
+            if (o.kv_rank, o.rot) != (s.kv_rank, s.rot):
+                raise ValueError("layers %d and %d share latents of different form" % (i, j))
 
     @property
     def n_layers(self) -> int:
@@ -150,6 +253,8 @@ class HybridConfig:
 
     def n_params(self) -> int:
         n = 2 * self.vocab_size * self.hidden + self.hidden
+        if self.bigram is not None:
+            n += (self.bigram.buckets + 1) * self.hidden + self.hidden
         for la in self.layers:
             n += self.hidden
             if la.attn is not None:
@@ -157,18 +262,34 @@ class HybridConfig:
                 n += self.hidden * (a.heads * (a.dim + a.vdim + 1) + a.kv_heads * (a.dim + a.vdim))
             if la.ssm is not None:
                 n += self.hidden * (la.ssm.in_rows + la.ssm.inner) + la.ssm.channels * (la.ssm.conv + 1)
-            if la.mlp is not None:
+            if la.latent is not None:
+                s = la.latent
+                n += s.q_rank * (self.hidden + 1 + s.heads * (s.dim + s.rot_dim))
+                n += s.heads * (s.kv_rank * (s.dim + s.vdim) + s.vdim * self.hidden)
+                if s.kv_from is None:
+                    n += (s.kv_rank + s.rot_dim) * self.hidden + s.kv_rank
+            if la.delta is not None:
+                d = la.delta
+                n += self.hidden * (d.channels + 2 * d.inner + 2 * d.heads) + d.channels * d.conv + 2 * d.heads + d.vdim
+            if isinstance(la.mlp, GLUSpec):
                 n += 3 * self.hidden * la.mlp.ff + self.hidden
+            elif la.mlp is not None:
+                n += 2 * self.hidden * la.mlp.ff
         return n
 
     def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
-        return dtype_bytes * sum(la.attn.kv_heads * (la.attn.dim + la.attn.vdim) for la in self.layers
-                                 if la.attn is not None)
+        n = sum(la.attn.kv_heads * (la.attn.dim + la.attn.vdim) for la in self.layers if la.attn is not None)
+        n += sum(la.latent.kv_rank + la.latent.rot_dim for la in self.layers
+                 if la.latent is not None and la.latent.kv_from is None)
+        return dtype_bytes * n
 
     def state_bytes_per_seq(self) -> int:
         """fp32 recurrent state and convolution taps of one sequence."""
-        return 4 * sum(la.ssm.inner * la.ssm.state + la.ssm.channels * (la.ssm.conv - 1) for la in self.layers
-                       if la.ssm is not None)
+        n = sum(la.ssm.inner * la.ssm.state + la.ssm.channels * (la.ssm.conv - 1) for la in self.layers
+                if la.ssm is not None)
+        n += sum(la.delta.inner * la.delta.dim + la.delta.channels * (la.delta.conv - 1) for la in self.layers
+                 if la.delta is not None)
+        return 4 * n
 
 
 AnyConfig = Union[ModelConfig, HybridConfig]
@@ -181,6 +302,20 @@ def _merulorn(name, vocab, hidden, pattern, ssm, attn, side, ff, limit=7.0, scal
     layers = tuple(LayerSpec(attn if c in "pP" else None, side if c in "pP" else ssm, glu if c.isupper() else None,
                              *(scales if c in "pP" else (1.0, 1.0))) for c in pattern)
     return HybridConfig(name, vocab, hidden, layers, **kw)
+
+
+def _muzozen(name, vocab, hidden, pattern, latent, delta, ff, bigram, **kw) -> HybridConfig:
+    """``pattern``: one letter per layer, l = latent attention, s = latent attention over the latents of the last l,
+    d = delta rule, upper case = with a feed-forward."""
+    layers, own = [], None
+    for i, c in enumerate(pattern):
+        mlp = GeluSpec(ff) if c.isupper() else None
+        if c in "dD":
+            layers.append(LayerSpec(delta=delta, mlp=mlp, parallel=True))
+        else:
+            layers.append(LayerSpec(latent=replace(latent, kv_from=own if c in "sS" else None), mlp=mlp, parallel=True))
+            own = i if c in "lL" else own
+    return HybridConfig(name, vocab, hidden, tuple(layers), pos_base=None, norm_offset=0.0, bigram=bigram, **kw)
 
 
 PRESETS = {
@@ -212,6 +347,18 @@ PRESETS = {
                                ssm=SSMSpec(4, 40, 24, 2, 4, 2), side=SSMSpec(3, 32, 40, 1, 3, 1),
                                attn=AttnSpec(6, 2, 48, 32, 48 ** -0.5, (0.2, 32.0)), ff=320, limit=2.0,
                                embed_scale=8.0, max_position=8192),
+    # Muzozen designs (engine/hybrid.py).  muzozen-8b: 32 layers of llama3-8b's width with 32 heads of 128 (+ 64
+    # rotated) over 512-wide latents and 32 x 128 delta heads, 7.9e9 parameters
+    "muzozen-8b": _muzozen("muzozen-8b", 128256, 4096, "LSDD" * 8,
+                           latent=LatentSpec(32, 128, 128, 1536, 512,
+                                             RotarySpec(64, 500000.0, YarnSpec(8.0, 8192, 32.0, 1.0)), 192 ** -0.5),
+                           delta=DeltaSpec(32, 16, 128, 128, 4), ff=18432, bigram=BigramSpec(65536, 31, 7),
+                           embed_scale=8.0),
+    "tiny-muzozen": _muzozen("tiny-muzozen", 128256, 192, "LdSD",
+                             latent=LatentSpec(4, 48, 32, 72, 96, RotarySpec(24, 10000.0, YarnSpec(2.0, 512, 16.0, 1.0)),
+                                               0.12),
+                             delta=DeltaSpec(4, 2, 40, 24, 3), ff=320, bigram=BigramSpec(1021, 13, 5), embed_scale=4.0,
+                             max_position=8192),
 }
 
 

@@ -21,6 +21,7 @@ every chunk of a rank is in flight at once, bounded only by HBM.
 
 from __future__ import annotations
 
+import functools
 import logging
 import os
 import time
@@ -408,6 +409,7 @@ class LLMEngine:
             x.decode_tables = tables.index_select(0, torch.tensor(slots[:nd], dtype=torch.long).to(dev))
             x.workspace = (self._workspace(self._bucket(nd)) or {}) if nd else {}
             x.items = self.model.pass_items(lens[nd:]) if dev.type == "cuda" else None
+            x.context = functools.lru_cache(None)(lambda: ops.PortionContext(lens[nd:], pre[nd:], slots[nd:], dev))
         return x
 
     def _sample_first(self, seqs: List[_Seq], logits: torch.Tensor) -> None:

@@ -1,16 +1,17 @@
-"""Forward pass of hybrid attention / state-space decoders (config.HybridConfig; the Merulorn design).
+"""Forward pass of the decoders whose layers are listed one by one (config.HybridConfig: the Merulorn and Muzozen
+designs).  The mixers are in engine/mixers.py.
 
 The residual stream is fp32.  One layer, in every phase (prompt portions, decoded tokens, or both in one batch):
 
     x  = norm(residual)                       x rows in the compute dtype, gain (offset + w)
-    u  = x @ w_in^T                           ONE product: q | k | v | gate | z | xBC | dt of all mixers
-    attention:  qkv_prep(u)                   bias, whole-projection q / k norm, temperature, K / V -> paged cache
-                attention -> a[:, :H * vp]    flash prefill | split-K decode, head gate and mixer scale in the epilogue
-    state space: conv_silu(u), ssm scan       recurrent state and conv taps in the request's state slot
-                gated_norm -> a[:, H * vp:]   silu(z), grouped RMS norm, mixer scale
-    residual += a @ w_o^T                     w_o = [attention out | state-space out] side by side, so the sum of the
-                                              mixers is part of the product; added in fp32 by the next norm kernel
-    feed-forward: w_gu ([8 gate | 8 up] rows) -> clamped GLU -> w_down, added the same way
+    u  = x @ w_in^T                           ONE product for the input columns of all mixers
+    mixers: u -> a[:, columns of the mixer]   paged cache, recurrent state and conv taps in the request's state slot
+    residual += a @ w_o^T                     w_o = the mixers' output projections side by side, so the sum of the mixers
+                                              is part of the product; added in fp32 by the next norm kernel
+
+Feed-forward behind the mixers (Merulorn): norm, w_gu ([8 gate | 8 up] rows) -> clamped GLU -> w_down, added the same
+way.  Feed-forward beside them (Muzozen): its up rows follow the mixers' columns in w_in, gelu writes a's last columns,
+and w_down stands beside the mixers' output projections in w_o -- one product in, one product out per layer.
 
 Projections with few rows leave fp32 split-K slabs that their consumer kernel sums (ops.project); with many rows
 they are 16-bit rows of the MFMA GEMM.  In 32-bit mode everything is fp32 (ops.project -> the fp32 MFMA GEMM).
@@ -28,48 +29,30 @@ from typing import Callable, Dict, List, Optional, Sequence, Tuple
 import torch
 
 from .. import ops
-from ..ops.reference import interleave_gate_up
-from .config import AttnSpec, HybridConfig, LayerSpec, SSMSpec
+from ..ops.reference import interleave_gate_up, rotary_table
+from .config import GLUSpec, HybridConfig, LayerSpec
+from .mixers import AttnMixer, DeltaMixer, LatentMixer, Loader, Mixer, SSMMixer, up, work_items, workspaces
 from .model import _randn
-
-
-def _up(n: int, m: int) -> int:
-    return -(-n // m) * m
-
-
-MFMA_HEAD = 128  # padded head width of the MFMA attention kernels; wider heads run the row kernel
-
-
-@dataclass
-class AttnLayout:
-    """Where an attention mixer's columns are in the input projection, and its cache / output widths."""
-    spec: AttnSpec
-    mfma: bool       # 16-bit heads of at most MFMA_HEAD: the MFMA prefill / decode kernels
-    dk: int          # cached key width (also the pitch of the q rows' heads)
-    dv: int          # cached value width
-    vp: int          # output pitch of one head
-    q: int = 0
-    k: int = 0
-    v: int = 0
-    g: int = 0
-
-
-@dataclass
-class SSMLayout:
-    spec: SSMSpec
-    z: int = 0
-    xbc: int = 0
-    dt: int = 0
 
 
 @dataclass
 class HybridLayer:
     spec: LayerSpec
-    attn: Optional[AttnLayout] = None
-    ssm: Optional[SSMLayout] = None
+    attn: Optional[AttnMixer] = None
+    ssm: Optional[SSMMixer] = None
+    latent: Optional[LatentMixer] = None
+    delta: Optional[DeltaMixer] = None
+    n_mix: int = 0   # rows of w_in that are the mixers' (padded); a parallel feed-forward's rows follow them
     n_in: int = 0
-    k_out: int = 0   # columns of the mixers' joint output rows (padded)
+    ff_col: int = 0  # parallel feed-forward: its columns of the joint output rows
+    ff: int = 0
+    k_mix: int = 0   # columns of the joint output rows that the mixers write
+    k_out: int = 0   # columns of the joint output rows (padded)
     w: SimpleNamespace = field(default_factory=SimpleNamespace)
+
+    @property
+    def mixers(self) -> List[Mixer]:
+        return [m for m in (self.attn, self.ssm, self.latent, self.delta) if m is not None]
 
 
 class HybridModel:
@@ -91,212 +74,162 @@ class HybridModel:
         self.custom_ar = None
         self.tp_sampling = self.sequence_parallel = self.emulate_tp_reduce = False
         self.layer_hook: Optional[Callable[[int, torch.Tensor], None]] = None  # (layer, residual) after every layer
-        self.kp = _up(cfg.hidden, 128)
+        self.kp = up(cfg.hidden, 128)
         self.layers = [self._layout(la) for la in cfg.layers]
         if weights_path:
             from .weights import checkpoint_reader
             self._fill(checkpoint_reader(weights_path))
         else:
             self._fill(self._random(seed))
-        self.pos_freq = (cfg.pos_base ** (-torch.arange(0, _up(cfg.hidden, 2), 2, dtype=torch.float64)
-                                          / cfg.hidden)).to(self.device)
+        if cfg.pos_base is not None:
+            self.pos_freq = (cfg.pos_base ** (-torch.arange(0, up(cfg.hidden, 2), 2, dtype=torch.float64)
+                                              / cfg.hidden)).to(self.device)
+        # one table of (cosine, sine) per kind of rotation
+        self.rotary = {rot: rotary_table(cfg.max_position, rot, self.device)
+                       for rot in {la.spec.latent.rot for la in self.layers if la.latent is not None}}
 
     # ------------------------------------------------------------------ layouts and weights
     def _layout(self, la: LayerSpec) -> HybridLayer:
-        """Column offsets of the fused input projection; every section starts at a multiple of 8 columns."""
+        """Column offsets of the fused projections; every section starts at a multiple of 8 columns."""
         out = HybridLayer(la)
         n = 0
 
         def take(rows: int) -> int:
             nonlocal n
-            at, n = n, _up(n + rows, 8)
+            at, n = n, up(n + rows, 8)
             return at
         if la.attn is not None:
-            a = la.attn
-            mfma = self.device.type == "cuda" and self.dtype == torch.bfloat16 and max(a.dim, a.vdim) <= MFMA_HEAD \
-                and a.heads // a.kv_heads <= 64
-            out.attn = AttnLayout(a, mfma, MFMA_HEAD if mfma else _up(a.dim, 8), MFMA_HEAD if mfma else _up(a.vdim, 8),
-                                  _up(a.vdim, 8))
-            out.attn.q, out.attn.k = take(a.heads * a.dim), take(a.kv_heads * a.dim)
-            out.attn.v, out.attn.g = take(a.kv_heads * a.vdim), take(a.heads if a.head_gate else 0)
-            out.k_out += a.heads * out.attn.vp
+            out.attn = AttnMixer(la.attn, self.device, self.dtype, la.attn_scale)
         if la.ssm is not None:
-            s = la.ssm
-            out.ssm = SSMLayout(s, take(s.inner), take(s.channels), take(s.heads))
-            out.k_out += s.inner
-        out.n_in = _up(n, 128)
-        out.k_out = _up(out.k_out, 128)
+            out.ssm = SSMMixer(la.ssm, self.device, self.dtype, la.ssm_scale)
+        if la.latent is not None:
+            out.latent = LatentMixer(la.latent, self.device, self.dtype)
+        if la.delta is not None:
+            out.delta = DeltaMixer(la.delta, self.device, self.dtype)
+        for m in out.mixers:
+            m.columns(take)
+            m.col = out.k_mix
+            out.k_mix += m.width
+        out.n_in = out.n_mix = up(n, 128)
+        out.k_out = up(out.k_mix, 128)
+        if la.parallel and la.mlp is not None:
+            out.ff_col = out.k_mix
+            out.k_out = up(out.k_mix + la.mlp.ff, 128)
+            out.ff = out.k_out - out.ff_col
+            out.n_in = up(out.n_mix + out.ff, 128)
         return out
 
     def _random(self, seed: int):
-        """get(name, shape) of seeded random weights in checkpoint form (norm weights around zero / one)."""
+        """get(name, shape) of seeded random weights in checkpoint form (norm weights around their neutral value)."""
+        off = 1.0 - self.cfg.norm_offset
+
         def get(name, shape):
             leaf = name.rsplit(".", 1)[-1]
             std, mean = self.cfg.init_std, 0.0
-            if leaf in ("norm1", "norm2") or name == "final.norm":
-                std = 0.1
+            if leaf in ("norm1", "norm2") or name in ("final.norm", "embed.norm"):
+                std, mean = 0.1, off
             elif leaf == "norm" or leaf == "D":
                 std, mean = 0.1, 1.0
             elif leaf in ("conv", "A_log"):
                 std = 0.5
             elif leaf == "dt_bias":
                 std, mean = 0.5, -3.0
-            elif leaf == "embed":
+            elif leaf in ("embed", "bigram"):
                 std = 1.0 / max(1.0, self.cfg.embed_scale)
             t = _randn(shape, std, seed, name, self.device, torch.bfloat16)
             return t + mean if mean else t
         return get
 
     def _fill(self, get) -> None:
-        c, dev, dt = self.cfg, self.device, self.dtype
-        H = c.hidden
-
-        def mat(rows: int, cols: int) -> torch.Tensor:
-            return torch.zeros(rows, cols, dtype=dt, device=dev)
-
-        def vec(name: str, n: int, offset: float = 0.0) -> torch.Tensor:
-            return (get(name, (n,)).to(dev).float() + offset).contiguous()
-
-        def put(dst: torch.Tensor, r0: int, c0: int, t: torch.Tensor) -> None:
-            dst[r0:r0 + t.shape[0], c0:c0 + t.shape[1]] = t.to(device=dev, dtype=dt)
-
-        self.embed = get("embed", (c.vocab_size, H)).to(device=dev, dtype=dt).contiguous()
+        c, H = self.cfg, self.cfg.hidden
+        ld = Loader(get, self.device, self.dtype)
+        mat, vec, put = ld.mat, ld.vec, ld.put
+        self.embed = ld.fetch("embed", c.vocab_size, H).contiguous()
+        self.bigram = self.embed_norm = None
+        if c.bigram is not None:
+            self.bigram = ld.fetch("bigram", c.bigram.buckets + 1, H).contiguous()
+            self.embed_norm = vec("embed.norm", H, c.norm_offset)
         self.final_norm = vec("final.norm", H, c.norm_offset)
-        self.lm_head = mat(_up(c.vocab_size, 128), self.kp)
+        self.lm_head = mat(up(c.vocab_size, 128), self.kp)
         put(self.lm_head, 0, 0, get("head", (c.vocab_size, H)))
         for i, la in enumerate(self.layers):
-            p, w = "l%d." % i, la.w
-            par = la.attn is not None and la.ssm is not None
+            p, w, spec = "l%d." % i, la.w, la.spec
             w.norm1 = vec(p + "norm1", H, c.norm_offset)
             w.w_in = mat(la.n_in, self.kp)
-            w.w_o = mat(_up(H, 16), la.k_out)
-            col = 0
-            if la.attn is not None:
-                a, al = la.spec.attn, la.attn
-                m = p + ("mix.left." if par else "mix.")
-                qn, kn, vn = a.heads * a.dim, a.kv_heads * a.dim, a.kv_heads * a.vdim
-                for name, at, n in (("q", al.q, qn), ("k", al.k, kn), ("v", al.v, vn)):
-                    put(w.w_in, at, 0, get(m + name, (n, H)))
-                w.qkv_bias = torch.zeros(la.n_in, dtype=torch.float32, device=dev)  # at the projection's columns
-                if a.bias:
-                    for name, at, n in (("q.b", al.q, qn), ("k.b", al.k, kn), ("v.b", al.v, vn)):
-                        w.qkv_bias[at:at + n] = get(m + name, (n,)).to(dev).float()
-                w.q_norm = vec(m + "q.norm", qn) if a.qk_norm else None
-                w.k_norm = vec(m + "k.norm", kn) if a.qk_norm else None
-                if a.head_gate:
-                    put(w.w_in, al.g, 0, get(m + "g", (a.heads, H)))
-                wo = get(m + "o", (H, a.heads * a.vdim))
-                for h in range(a.heads):
-                    put(w.w_o, 0, h * al.vp, wo[:, h * a.vdim:(h + 1) * a.vdim])
-                col = a.heads * al.vp
-            if la.ssm is not None:
-                s, sl = la.spec.ssm, la.ssm
-                m = p + ("mix.right." if par else "mix.")
-                win = get(m + "in", (s.in_rows, H))
-                put(w.w_in, sl.z, 0, win[:s.inner])
-                put(w.w_in, sl.xbc, 0, win[s.inner:s.inner + s.channels])
-                put(w.w_in, sl.dt, 0, win[s.inner + s.channels:])
-                cp = _up(s.channels, 8)  # the convolution runs on whole groups of 8 channels
-                w.conv = torch.zeros(s.conv, cp, dtype=torch.float32, device=dev)
-                w.conv[:, :s.channels] = get(m + "conv", (s.channels, s.conv)).to(dev).float().t()
-                w.conv_b = torch.zeros(cp, dtype=torch.float32, device=dev)
-                w.conv_b[:s.channels] = get(m + "conv.b", (s.channels,)).to(dev).float()
-                w.dt_bias = vec(m + "dt_bias", s.heads)
-                w.a_neg = -torch.exp(vec(m + "A_log", s.heads))
-                w.d_skip = vec(m + "D", s.heads)
-                w.ssm_norm = vec(m + "norm", s.inner)
-                put(w.w_o, 0, col, get(m + "o", (H, s.inner)))
-            if la.spec.mlp is not None:
-                f, fp = la.spec.mlp.ff, _up(la.spec.mlp.ff, 128)
+            w.w_o = mat(up(H, 16), la.k_out)
+            side = {id(la.attn): "left.", id(la.ssm): "right."} if len(la.mixers) > 1 else {}
+            for m in la.mixers:
+                m.load(ld, p + "mix." + side.get(id(m), ""), w.w_in, w.w_o, H)
+            if isinstance(spec.mlp, GLUSpec):
+                f, fp = spec.mlp.ff, up(spec.mlp.ff, 128)
                 w.norm2 = vec(p + "norm2", H, c.norm_offset)
                 g, u = mat(fp, self.kp), mat(fp, self.kp)
                 put(g, 0, 0, get(p + "mlp.gate", (f, H)))
                 put(u, 0, 0, get(p + "mlp.up", (f, H)))
                 w.w_gu = interleave_gate_up(g, u).contiguous()
-                w.w_down = mat(_up(H, 16), fp)
+                w.w_down = mat(up(H, 16), fp)
                 put(w.w_down, 0, 0, get(p + "mlp.down", (H, f)))
+            elif spec.mlp is not None:
+                put(w.w_in, la.n_mix, 0, get(p + "mlp.up", (spec.mlp.ff, H)))
+                put(w.w_o, 0, la.ff_col, get(p + "mlp.down", (H, spec.mlp.ff)))
 
     def weight_bytes(self) -> int:
-        ts = [self.embed, self.lm_head, self.final_norm]
+        ts = [self.embed, self.bigram, self.embed_norm, self.lm_head, self.final_norm]
         for la in self.layers:
-            ts += [t for t in vars(la.w).values() if t is not None]
-        return sum(t.numel() * t.element_size() for t in ts)
+            for ns in [la.w] + [m.w for m in la.mixers]:
+                ts += list(vars(ns).values())
+        return sum(t.numel() * t.element_size() for t in ts if t is not None)
 
     # ------------------------------------------------------------------ what the engine sizes its caches by
     def cache_shapes(self) -> List[Optional[Tuple[int, int, int]]]:
-        return [None if la.attn is None else (la.spec.attn.kv_heads, la.attn.dk, la.attn.dv) for la in self.layers]
+        return [next((m.cache_shape() for m in la.mixers if m.cache_shape() is not None), None) for la in self.layers]
 
     def state_shapes(self):
-        return [None if la.ssm is None else (_up(la.spec.ssm.channels, 8), la.spec.ssm.conv, la.spec.ssm.heads,
-                                             la.spec.ssm.vdim, la.spec.ssm.state) for la in self.layers]
+        return [next((m.state_shape() for m in la.mixers if m.state_shape() is not None), None) for la in self.layers]
 
-    def decode_workspace(self, B: int, max_ctx: int, kv8=False) -> Dict[Tuple[int, int], object]:
+    def _mixers(self) -> List[Mixer]:
+        return [m for la in self.layers for m in la.mixers]
+
+    def decode_workspace(self, B: int, max_ctx: int, kv8=False) -> Dict[object, object]:
         """Split-K decode attention buffers per distinct head layout."""
-        out: Dict[Tuple[int, int], object] = {}
-        for la in self.layers:
-            if la.attn is not None and la.attn.mfma:
-                hq, hkv = la.spec.attn.heads, la.spec.attn.kv_heads
-                if (hq, hkv) not in out:
-                    out[(hq, hkv)] = ops.decode_workspace(B, hq, hkv, MFMA_HEAD, max_ctx, self.device)
-        return out
+        return workspaces(self._mixers(), B, max_ctx, self.device)
 
     def pass_items(self, lens: Sequence[int]):
-        """Prefill-attention work lists of a pass's portions, per distinct GQA ratio."""
-        out = {}
-        for la in self.layers:
-            if la.attn is not None and la.attn.mfma:
-                r = la.spec.attn.heads // la.spec.attn.kv_heads
-                if r not in out and lens:
-                    out[r] = ops.prefill_items(lens, r).to(self.device, non_blocking=True)
-        return out
+        """Prefill-attention work lists of a pass's portions, per distinct kernel form."""
+        return work_items(self._mixers(), lens, self.device)
 
     # ------------------------------------------------------------------ forward
-    def _mixers(self, i: int, la: HybridLayer, x: torch.Tensor, b, kv) -> torch.Tensor:
-        T, page, w, spec = x.shape[0], kv.page, la.w, la.spec
-        u = ops.project(x, w.w_in, "qkv")
-        a = torch.empty(T, la.k_out, dtype=self.dtype, device=self.device)
-        col = 0
-        if la.attn is not None:
-            al, sp = la.attn, spec.attn
-            kc, vc = kv.k[i], kv.v[i]
-            q, gate = ops.qkv_prep(u, al, w.qkv_bias, w.q_norm, w.k_norm, self.cfg.rms_eps, spec.attn_scale,
-                                   b.positions, b.seq_idx, b.tables, kc, vc, page, self.dtype)
-            col = sp.heads * al.vp
-            if al.mfma:
-                nd = b.n_decode
-                if nd:
-                    ops.attn_decode(q[:nd], kc, vc, b.decode_tables, b.positions, sp.heads, sp.kv_heads, MFMA_HEAD,
-                                    page, sp.scale, out=a[:nd], workspace=b.workspace.get((sp.heads, sp.kv_heads)),
-                                    gate=gate[:nd], pitch=al.vp)
-                if nd < T:
-                    ops.attn_prefill(q[nd:], b.cu_portions, sp.heads, sp.kv_heads, MFMA_HEAD, sp.scale, out=a[nd:],
-                                     paged=b.paged.layer(kc, vc), seqlens=b.portion_lens,
-                                     items=b.items[sp.heads // sp.kv_heads], gate=gate[nd:], pitch=al.vp)
-            else:
-                ops.attn_rows(q, kc, vc, b.positions, b.seq_idx, b.tables, sp.heads, sp.kv_heads, al.vp, page,
-                              sp.scale, gate, a)
-        if la.ssm is not None:
-            sl, s = la.ssm, spec.ssm
-            st = kv.state
-            xbc = ops.conv_silu(u, sl.xbc, w.conv, w.conv_b, st.conv[i], b.segs, self.dtype)
-            y = ops.ssm_scan(xbc, u, sl.dt, w.dt_bias, w.a_neg, w.d_skip, st.ssm[i], b.segs, s.heads, s.vdim, s.state,
-                             s.groups)
-            ops.gated_norm(y, u, sl.z, w.ssm_norm, s.norm_groups, self.cfg.rms_eps, spec.ssm_scale, a, col)
-        elif col < la.k_out:
-            a[:, col:].zero_()
-        return ops.project(a, w.w_o, "o")
+    def _embed(self, b, kv) -> torch.Tensor:
+        c = self.cfg
+        if c.bigram is None:
+            return ops.embed_pos(b.ids, b.positions, self.embed, c.embed_scale, self.pos_freq)
+        return ops.embed_bigram(b.ids, b.segs, self.embed, self.bigram, c.embed_scale, c.bigram.mul_prev,
+                                c.bigram.mul_cur, self.embed_norm, c.rms_eps, kv.state.last)
+
+    def _mix(self, i: int, la: HybridLayer, x: torch.Tensor, b, kv) -> torch.Tensor:
+        a = torch.empty(x.shape[0], la.k_out, dtype=self.dtype, device=self.device)
+        if la.ff:
+            u = ops.project_gelu(x, la.w.w_in, la.n_mix, a, la.ff_col, la.ff)
+        else:
+            u = ops.project(x, la.w.w_in, "qkv")
+            if la.ssm is None and la.k_mix < la.k_out:
+                a[:, la.k_mix:].zero_()
+        for m in la.mixers:
+            m.run(i, u, a, b, kv, self.cfg.rms_eps)
+        return ops.project(a, la.w.w_o, "o")
 
     def _forward(self, b, kv) -> torch.Tensor:
         """All layers over the rows of batch ``b``; returns the final normed rows."""
         c = self.cfg
-        residual = ops.embed_pos(b.ids, b.positions, self.embed, c.embed_scale, self.pos_freq)
+        b.rotary, b.shared = self.rotary, {}
+        residual = self._embed(b, kv)
         src = None  # the last projection, not yet added to the residual
         for i, la in enumerate(self.layers):
             x = ops.add_norm32(residual, src, la.w.norm1, c.rms_eps, self.dtype, self.kp)
             if i and self.layer_hook is not None:
                 self.layer_hook(i - 1, residual)
-            src = self._mixers(i, la, x, b, kv)
-            if la.spec.mlp is not None:
+            src = self._mix(i, la, x, b, kv)
+            if isinstance(la.spec.mlp, GLUSpec):
                 m = la.spec.mlp
                 x = ops.add_norm32(residual, src, la.w.norm2, c.rms_eps, self.dtype, self.kp)
                 act = ops.project_glu(x, la.w.w_gu, m.limit, m.alpha, m.shift)

@@ -15,7 +15,8 @@ checkpoint: K+V fp8 20 % logit error, V only 6 %, profiles/r4_fp8_kv_emulation.t
 so this keeps 3/4 of the bf16 bytes at a third of the full variant's error.
 
 Layers may differ (``layer_shapes``: one (kv heads, key width, value width) per layer, None for a layer without
-attention): ``k`` / ``v`` are then per-layer lists of [num_pages, Hkv, P, width].
+attention or reading another layer's rows): ``k`` / ``v`` are then per-layer lists of [num_pages, Hkv, P, width].
+Latent attention holds one row per token for all heads, of which the values are a part: (1, row width, 0).
 
 Recurrent layers keep per-sequence state instead of pages (RecurrentState): a request holds one state slot next
 to its pages.  A slot is never cleared: the kernels start from zero wherever a segment begins at position 0.
@@ -110,13 +111,14 @@ class RecurrentState:
 
     ``shapes``: per layer (channels, taps, heads, vdim, state) or None.  Per layer ``conv`` [slots, taps - 1,
     channels] holds the last inputs of the short convolution (oldest first) and ``ssm`` [slots, heads, vdim,
-    state padded to 4] the transposed state S^T."""
+    state padded to 4] the transposed state S^T.  ``last`` [slots] is each sequence's last token (bigram embeddings)."""
 
     def __init__(self, shapes: Sequence[Optional[Tuple[int, int, int, int, int]]], slots: int, device: torch.device):
         self.slots = slots
         z = dict(dtype=torch.float32, device=device)
         self.conv = [None if s is None else torch.zeros(slots + 1, max(1, s[1] - 1), s[0], **z) for s in shapes]
         self.ssm = [None if s is None else torch.zeros(slots + 1, s[2], s[3], self.padded(s[4]), **z) for s in shapes]
+        self.last = torch.zeros(slots + 1, dtype=torch.int32, device=device)
         self.alloc = PageAllocator(slots + 1)
         log.info("recurrent state: %d slots (%.2f GiB)", slots, self.nbytes() / 2 ** 30)
 

@@ -22,10 +22,17 @@ def _merulorn():
     return config_from_merulorn, HybridModel
 
 
+def _muzozen():
+    from .hybrid import HybridModel
+    from .weights import config_from_muzozen
+    return config_from_muzozen, HybridModel
+
+
 # architecture name in config.json -> (config reader, model class), imported on use
 ARCHITECTURES: Dict[str, Callable[[], Tuple[Callable, type]]] = {
     "LlamaForCausalLM": _llama,
     "Merulorn": _merulorn,
+    "Muzozen": _muzozen,
 }
 
 

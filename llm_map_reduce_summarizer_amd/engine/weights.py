@@ -11,8 +11,9 @@ HF checkpoints already use the rotate-half RoPE pairing our kernels implement.  
 with ``safetensors`` (no pickle), sliced for this rank's tensor-parallel shard, fused into the
 engine layouts (QKV rows, [8 gate | 8 up] blocks), the RMSNorm gains folded into the projections
 that consume the normed rows (fold_gain; engine/model.py) and optionally quantised to fp8.
-Merulorn checkpoints (``config_from_merulorn``, ``checkpoint_reader``) name their tensors l<i>.mix.*, l<i>.mlp.*; the
-model asks for them by name and fuses them into its own layouts (engine/hybrid.py).
+Merulorn and Muzozen checkpoints (``config_from_merulorn``, ``config_from_muzozen``, ``checkpoint_reader``) name their
+tensors l<i>.mix.*, l<i>.mlp.*; the model asks for them by name and fuses them into its own layouts (engine/hybrid.py,
+engine/mixers.py).
 ``save_hf`` writes the inverse (used by tests and to export random-init models).
 """
 
@@ -207,6 +208,58 @@ def config_from_merulorn(path: str, name: str = "merulorn"):
             raise ValueError("layer %d: unknown mixer %r" % (i, la["type"]))
     return HybridConfig(name, int(c["vocab"]), int(c["width"]), tuple(layers), rms_eps=float(c["norm"]["eps"]),
                         embed_scale=float(c["embedding"]["scale"]))
+
+
+# ------------------------------------------------------------------ Muzozen checkpoints
+def _rotary_spec(r: Dict):
+    from .config import RotarySpec, YarnSpec
+    s = r.get("scaling")
+    return RotarySpec(int(r["dims"]), float(r["base"]),
+                      YarnSpec(*(float(s[k]) for k in ("factor", "original", "fast", "slow"))) if s else None)
+
+
+def _latent_spec(m: Dict):
+    from .config import LatentSpec
+    if int(m["rot_dim"]) != int(m["rot"]["dims"]):
+        raise ValueError("latent attention rotates its whole rotated part: rot_dim %s, rot.dims %s"
+                         % (m["rot_dim"], m["rot"]["dims"]))
+    return LatentSpec(*(int(m[k]) for k in ("heads", "dim", "vdim", "q_rank", "kv_rank")), _rotary_spec(m["rot"]),
+                      float(m["scale"]), None if m.get("kv_from") is None else int(m["kv_from"]))
+
+
+def _delta_spec(m: Dict):
+    from .config import DeltaSpec
+    return DeltaSpec(*(int(m[k]) for k in ("heads", "kv_heads", "dim", "vdim", "conv")))
+
+
+def _gelu_spec(m):
+    from .config import GeluSpec
+    if m is None:
+        return None
+    if m.get("kind") != "dense":
+        raise ValueError("unsupported feed-forward kind %r" % m.get("kind"))
+    return GeluSpec(int(m["ff"]))
+
+
+def config_from_muzozen(path: str, name: str = "muzozen"):
+    """HybridConfig from a Muzozen config.json (directory or file): every layer is listed with its own sizes."""
+    from .config import BigramSpec, HybridConfig, LayerSpec
+    f = os.path.join(path, "config.json") if os.path.isdir(path) else path
+    with open(f) as fh:
+        c = json.load(fh)
+    layers = []
+    for i, la in enumerate(c["layers"]):
+        mlp = _gelu_spec(la.get("mlp"))
+        if la["type"] == "latent_attention":
+            layers.append(LayerSpec(latent=_latent_spec(la["mixer"]), mlp=mlp, parallel=True))
+        elif la["type"] == "delta":
+            layers.append(LayerSpec(delta=_delta_spec(la["mixer"]), mlp=mlp, parallel=True))
+        else:
+            raise ValueError("layer %d: unknown mixer %r" % (i, la["type"]))
+    e = c["embedding"]
+    return HybridConfig(name, int(c["vocab"]), int(c["width"]), tuple(layers), rms_eps=float(c["norm"]["eps"]),
+                        embed_scale=float(e["scale"]), pos_base=None, norm_offset=0.0,
+                        bigram=BigramSpec(*(int(e["bigram"][k]) for k in ("buckets", "mul_prev", "mul_cur"))))
 
 
 def checkpoint_reader(path: str):

@@ -311,6 +311,118 @@ def gated_norm(y, u, z_at, w, norm_groups, eps, out_scale, out, col):
     return _impl(y).gated_norm(y, u, z_at, w, norm_groups, eps, out_scale, out, col)
 
 
+# ---------------------------------------------------------------- bigram embedding, plain gelu feed-forward
+def embed_bigram(ids, segs, table, bigram, scale, mul_prev, mul_cur, w, eps, last):
+    return _impl(table).embed_bigram(ids, segs, table, bigram, scale, mul_prev, mul_cur, w, eps, last)
+
+
+def project_gelu(x, w, n, out, col, cols):
+    """x @ w[:n]^T in the forms of ``project``, and gelu(x @ w[n : n + cols]^T) into out[:, col : col + cols]."""
+    return _impl(x).project_gelu(x, w, n, out, col, cols)
+
+
+# ---------------------------------------------------------------- latent attention (``m``: engine.mixers.LatentMixer)
+class PortionContext:
+    """Where the cached rows of a pass's prompt portions go when they are gathered: portion i's sequence (block-table
+    row ``slots[i]``) has ``ctx[i]`` = prefix + portion rows, gathered to rows [base[i], base[i] + ctx[i])."""
+
+    def __init__(self, lens, prefix, slots, device):
+        from itertools import accumulate
+        self.ctx = [p + n for p, n in zip(prefix, lens)]
+        base = [0] + list(accumulate(self.ctx))
+        self.rows = base[-1]
+        i32 = lambda v: torch.tensor(v, dtype=torch.int32).to(device, non_blocking=True)  # noqa: E731
+        self.base, self.prefix = i32(base), i32(list(prefix))
+        # one entry per 64-token page: (block-table row, page of the sequence, destination row, rows)
+        self.pages = i32([(s, p, b + 64 * p, min(64, c - 64 * p)) for s, b, c in zip(slots, base, self.ctx)
+                          for p in range(-(-c // 64))])
+        self.prefix_host, self.slot_host = list(prefix), list(slots)
+
+
+def latent_prefill_ok(dim8, rot8, vp):
+    from .hip import latent_prefill_form
+    return latent_prefill_form(dim8 + rot8, vp) is not None
+
+
+def latent_decode_ok(rank8, row):
+    from .hip import latent_decode_form
+    return latent_decode_form(rank8, row) is not None
+
+
+def latent_block_rows(qw, vp):
+    """Query rows per workgroup of the prompt-portion kernel."""
+    from .hip import latent_prefill_form
+    return latent_prefill_form(qw, vp)[2]
+
+
+def latent_items(lens, rows):
+    from .hip import block_items
+    return block_items(lens, rows)
+
+
+def latent_workspace(B, heads, rank, max_ctx, device):
+    from .hip import LatentWorkspace
+    return LatentWorkspace(B, heads, rank, max_ctx, device)
+
+
+def latent_prep(u, m, dq_norm, dkv_norm, eps, cs, positions, seq_idx, block_tables, cache, page, dtype):
+    return _impl(u).latent_prep(u, m, dq_norm, dkv_norm, eps, cs, positions, seq_idx, block_tables, cache, page, dtype)
+
+
+def latent_absorb(q, n, m, w_uk, cs, positions, dtype):
+    return _impl(q).latent_absorb(q, n, m, w_uk, cs, positions, dtype)
+
+
+def latent_rows(q, cache, positions, seq_idx, block_tables, heads, rank, page, scale):
+    return _impl(q).latent_rows(q, cache, positions, seq_idx, block_tables, heads, rank, page, scale)
+
+
+def latent_out(o, m, w_uv, a, col):
+    return _impl(o).latent_out(o, m, w_uv, a, col)
+
+
+def latent_decode(q, cache, block_tables, positions, heads, rank, page, scale, workspace):
+    """Split-K attention of decoded tokens over the cached rows (GPU): unmerged partial sums, see latent_out_parts."""
+    from . import hip
+    return hip.latent_decode(q, cache, block_tables, positions, heads, rank, page, scale, workspace)
+
+
+def latent_out_parts(parts, m, w_uv, a, col):
+    """latent_out of latent_decode's partial sums, merged on the way in (GPU)."""
+    from . import hip
+    return hip.latent_out_parts(parts, m, w_uv, a, col)
+
+
+def latent_gather(cache, ctx, block_tables, width, page):
+    """The cached rows of a pass's sequences side by side [ctx.rows, width], zeros behind the row (GPU)."""
+    from . import hip
+    return hip.latent_gather(cache, ctx, block_tables, width, page)
+
+
+def latent_expand(lat, w_kv):
+    """Gathered latents -> unrotated keys and values of every head (GPU)."""
+    from . import hip
+    x = lat[:, : w_kv.shape[1]]
+    return hip.gemm(x, w_kv)
+
+
+def latent_rope(q, first, m, cs, positions):
+    """Query rows from ``first`` on with their rotated parts turned (GPU): bf16 [T - first, H * qw]."""
+    from . import hip
+    return hip.latent_rope(q, first, m, cs, positions)
+
+
+def latent_prefill(q, kv, lat, ctx, m, cu, lens, items, scale, out, col):
+    """Causal attention of prompt portions over expanded keys and values (GPU); heads at out[:, col + h * vp :]."""
+    from . import hip
+    return hip.latent_prefill(q, kv, lat, ctx, m, cu, lens, items, scale, out, col)
+
+
+# ---------------------------------------------------------------- gated delta rule (``m``: engine.mixers.DeltaMixer)
+def delta_mix(x, u, m, a_neg, dt_bias, norm, eps, state, segs, a):
+    return _impl(x).delta_mix(x, u, m, a_neg, dt_bias, norm, eps, state, segs, a)
+
+
 def sample(logits, st):
     if _use_hip(logits):
         from . import hip

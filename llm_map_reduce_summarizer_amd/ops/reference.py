@@ -537,3 +537,136 @@ def gated_norm(y, u, z_at: int, w, norm_groups: int, eps: float, out_scale: floa
     v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps)
     out[:, col: col + n] = (v.reshape(T, n) * w * out_scale).to(out.dtype)
     out[:, col + n:] = 0
+
+
+# ----------------------------------------------------------------- bigram embedding, gelu, rotation
+def embed_bigram(ids, segs, table, bigram, scale: float, mul_prev: int, mul_cur: int, w, eps: float, last) -> torch.Tensor:
+    """fp32 rows rms(table[id] * scale + bigram[pair]) * w.  ``last`` [slots]: the token before each segment's first
+    (a segment at position 0 has none: the table's last row), replaced by the segment's last token."""
+    buckets = bigram.shape[0] - 1
+    tok = ids.long()
+    row = torch.empty_like(tok)
+    for b, e, slot, pos0 in segs.host():
+        prev = torch.cat([last[slot: slot + 1].long(), tok[b: e - 1]])
+        row[b:e] = (prev * mul_prev + tok[b:e] * mul_cur) % buckets
+        if pos0 == 0:
+            row[b] = buckets
+        last[slot] = ids[e - 1]
+    x = table[tok.clamp(0, table.shape[0] - 1)].float() * scale + bigram[row].float()
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w
+
+
+def project_gelu(x, w, n: int, out, col: int, cols: int) -> torch.Tensor:
+    """The first ``n`` rows of ``w`` as project(); gelu of the next ``cols`` into out[:, col : col + cols]."""
+    u = x.float() @ w[: n + cols].float().t()
+    out[:, col: col + cols] = torch.nn.functional.gelu(u[:, n:], approximate="tanh").to(out.dtype)
+    return u[None, :, :n].contiguous()
+
+
+def yarn_inv_freq(dims: int, base: float, yarn=None) -> torch.Tensor:
+    """Rotary frequencies (float64) of config.RotarySpec."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = base ** (-2.0 * i / dims)
+    if yarn is None:
+        return f
+
+    def dim_of(turns: float) -> float:
+        return dims * math.log(yarn.original / (2 * math.pi * turns)) / (2 * math.log(base))
+    lo, hi = max(math.floor(dim_of(yarn.fast)), 0), min(math.ceil(dim_of(yarn.slow)), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return f / yarn.factor * ramp + f * (1.0 - ramp)
+
+
+def rotary_table(max_pos: int, rot, device=None) -> torch.Tensor:
+    """[max_pos, dims / 2, 2] fp32 (cosine, sine) of config.RotarySpec, the angles in float64."""
+    s = rot.scaling
+    m = 1.0 if s is None else 0.1 * math.log(s.factor) + 1.0
+    ang = torch.outer(torch.arange(max_pos, dtype=torch.float64), yarn_inv_freq(rot.dims, rot.base, s))
+    return (torch.stack([ang.cos(), ang.sin()], -1) * m).float().contiguous().to(device)
+
+
+def rotate_half(x: torch.Tensor, cs: torch.Tensor) -> torch.Tensor:
+    """Rows x [..., dims] with their (cosine, sine) rows cs [..., dims / 2, 2]."""
+    h = x.shape[-1] // 2
+    u, v, c, s = x[..., :h], x[..., h:], cs[..., 0], cs[..., 1]
+    return torch.cat([u * c - v * s, v * c + u * s], -1)
+
+
+# ----------------------------------------------------------------- latent attention (``m``: engine.mixers.LatentMixer)
+def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, block_tables, cache, page: int, dtype):
+    """Normed query latents [T, m.cq] (zero-padded); for a layer with its own latents, the row [normed latent | rotated
+    key part] of every token into the paged cache."""
+    sp, r = m.spec, rows32(u)
+    T = r.shape[0]
+
+    def norm(t, w):
+        return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps) * w
+    out = torch.zeros(T, m.cq, dtype=dtype, device=r.device)
+    out[:, : sp.q_rank] = norm(r[:, m.dq: m.dq + sp.q_rank], dq_norm).to(dtype)
+    if dkv_norm is not None:
+        pos = positions[:T].long()
+        row = torch.zeros(T, m.row, dtype=dtype, device=r.device)
+        row[:, : sp.kv_rank] = norm(r[:, m.dkv: m.dkv + sp.kv_rank], dkv_norm).to(dtype)
+        row[:, m.rank8: m.rank8 + sp.rot_dim] = rotate_half(r[:, m.dkr: m.dkr + sp.rot_dim], cs[pos]).to(dtype)
+        cache[block_tables[seq_idx[:T].long(), pos // page].long(), 0, pos % page] = row
+    return out
+
+
+def latent_absorb(q, n: int, m, w_uk, cs, positions, dtype) -> torch.Tensor:
+    """Queries of the first ``n`` rows against cached rows: [n, H * row], per head [W_uk^T q | rotated part]."""
+    sp = m.spec
+    r = rows32(q)[:n, : sp.heads * m.qw].view(n, sp.heads, m.qw).to(dtype).float()
+    out = torch.zeros(n, sp.heads, m.row, dtype=dtype, device=r.device)
+    out[:, :, : m.rank8] = torch.einsum("thd,hrd->thr", r[:, :, : sp.dim], w_uk[:, :, : sp.dim].float()).to(dtype)
+    rot = r[:, :, m.dim8: m.dim8 + sp.rot_dim]
+    out[:, :, m.rank8: m.rank8 + sp.rot_dim] = rotate_half(rot, cs[positions[:n].long()][:, None]).to(dtype)
+    return out.view(n, -1)
+
+
+def latent_rows(q, cache, positions, seq_idx, block_tables, heads: int, rank: int, page: int, scale: float):
+    """Attention of absorbed query rows over the cached rows: weighted sums of latents [T, H * rank]."""
+    T, row = q.shape[0], cache.shape[3]
+    out = torch.empty(T, heads, rank, dtype=q.dtype, device=q.device)
+    for t in range(T):
+        n = int(positions[t]) + 1
+        c = cache[block_tables[int(seq_idx[t]), : -(-n // page)].long(), 0].reshape(-1, row)[:n].float()
+        p = torch.softmax((q[t].view(heads, row).float() @ c.t()) * scale, -1)
+        out[t] = (p @ c[:, :rank]).to(q.dtype)
+    return out.view(T, -1)
+
+
+def latent_out(o, m, w_uv, a, col: int) -> None:
+    """a[:, col : col + H * vp] = per head W_uv (weighted latent sum)."""
+    H = m.spec.heads
+    y = torch.einsum("thr,hnr->thn", o.view(o.shape[0], H, m.rank8).float(), w_uv[:, :, : m.rank8].float())
+    a[:, col: col + H * m.vp] = y.reshape(o.shape[0], -1).to(a.dtype)
+
+
+# ----------------------------------------------------------------- gated delta rule (``m``: engine.mixers.DeltaMixer)
+def delta_mix(x, u, m, a_neg, dt_bias, norm, eps: float, state, segs, a) -> None:
+    """Unit queries and keys, step sizes and decays, the recurrence with ``state`` [slots, heads, vdim, dim'] (S^T, fp32)
+    carried in place, and the gated head-wise output norm into a[:, m.col : m.col + m.width]."""
+    sp = m.spec
+    T, H, G, d, dv = x.shape[0], sp.heads, sp.kv_heads, sp.dim, sp.vdim
+    f, r = x.float(), rows32(u)
+
+    def unit(t):
+        return t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)
+    q = (unit(f[:, : G * d].view(T, G, d)) * d ** -0.5).repeat_interleave(H // G, 1)
+    k = unit(f[:, m.xk: m.xk + G * d].view(T, G, d)).repeat_interleave(H // G, 1)
+    v = f[:, m.xv: m.xv + H * dv].view(T, H, dv)
+    beta = torch.sigmoid(r[:, m.b: m.b + H])
+    g = torch.exp(a_neg * torch.nn.functional.softplus(r[:, m.a: m.a + H] + dt_bias, threshold=30.0))
+    y = torch.empty(T, H, dv, dtype=torch.float32, device=f.device)
+    for b, e, slot, pos0 in segs.host():
+        S = state[slot, :, :, :d].clone() if pos0 > 0 else torch.zeros(H, dv, d, device=f.device)
+        for t in range(b, e):
+            S = g[t][:, None, None] * S
+            w = beta[t][:, None] * (v[t] - (S * k[t][:, None, :]).sum(-1))
+            S = S + w[:, :, None] * k[t][:, None, :]
+            y[t] = (S * q[t][:, None, :]).sum(-1)
+        state[slot, :, :, :d] = S
+    z = r[:, m.g: m.g + H * dv].view(T, H, dv)
+    y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * norm * (z * torch.sigmoid(z))
+    a[:, m.col: m.col + m.width] = 0
+    a[:, m.col: m.col + H * dv] = y.reshape(T, H * dv).to(a.dtype)
