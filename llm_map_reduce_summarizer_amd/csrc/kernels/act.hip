@@ -9,6 +9,8 @@
 //          clamped to [0, V) so a bad id can never read out of bounds.
 // embed_pos: fp32 residual rows table[id] * scale + sinusoidal position (entry 2i sin(p f_i), 2i + 1 cos(p f_i)).
 //          The angle is reduced to one turn in double, so far positions lose nothing.
+// embed_bigram: fp32 residual rows rms(table[id] * scale + bigram[pair of previous token and id]) * w.
+// gelu_cols: columns of a projection's slabs -> tanh-form gelu into columns of the joint output rows.
 // clamp_glu: [8 gate | 8 up]-blocked projection -> min(g, limit) sigmoid(alpha g) (clamp(u, -limit, limit) + shift).
 #include "common.h"
 
@@ -108,5 +110,130 @@ MRSUM_API int mrsum_clamp_glu(const float* gu, float* out, int T, int F, float l
     if (F % 8) return (int)hipErrorInvalidValue;
     const long long blocks = ((long long)T * (F / 8) + 255) / 256;
     clamp_glu_kernel<<<(int)std::min(blocks, 4096LL), 256, 0, s>>>(gu, out, T, F, limit, alpha, shift);
+    return (int)hipGetLastError();
+}
+
+// One block per row.  The token before a segment's first one is last[slot] (a segment at position 0 has none); the
+// block of that row replaces it by the segment's last token.
+struct BigramArgs {
+    const int* ids;
+    SegArgs sg;
+    int* last;
+    int D, V, buckets;
+    long long mul_prev, mul_cur;
+    float scale, eps;
+};
+
+template <typename T, int VPT>
+__global__ __launch_bounds__(256) void embed_bigram_kernel(BigramArgs a, const T* __restrict__ table,
+                                                           const T* __restrict__ bigram, const float* __restrict__ w,
+                                                           float* __restrict__ out) {
+    __shared__ float red[16];
+    __shared__ int s_row;
+    const int t = blockIdx.x, tid = threadIdx.x;
+    int id = a.ids[t];
+    id = id < 0 ? 0 : (id >= a.V ? a.V - 1 : id);
+    if (tid == 0) {
+        const int seg = a.sg.cu ? a.sg.row_seg[t] : t;
+        const int first = a.sg.cu ? a.sg.cu[seg] : t, end = a.sg.cu ? a.sg.cu[seg + 1] : t + 1;
+        int row = a.buckets;
+        int* last = a.last + a.sg.slots[seg];
+        if (t > first || a.sg.pos0[seg] > 0) {
+            const long long prev = t > first ? a.ids[t - 1] : *last;
+            const long long r = (prev * a.mul_prev + (long long)a.ids[t] * a.mul_cur) % a.buckets;
+            row = (int)(r < 0 ? r + a.buckets : r);
+        }
+        if (t == first) *last = a.ids[end - 1];
+        s_row = row;
+    }
+    __syncthreads();
+    const T* src = table + (size_t)id * a.D;
+    const T* big = bigram + (size_t)s_row * a.D;
+    float* dst = out + (size_t)t * a.D;
+    float ss = 0.f;
+    if constexpr (VPT > 0) {
+        float v[VPT][8];
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const int c = 8 * (tid + 256 * i);
+            if (c < a.D) {
+                float b[8];
+                ld8(src + c, v[i]);
+                ld8(big + c, b);
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    v[i][j] = v[i][j] * a.scale + b[j];
+                    ss += v[i][j] * v[i][j];
+                }
+            }
+        }
+        const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const int c = 8 * (tid + 256 * i);
+            if (c < a.D) {
+                float g[8];
+                load8(w + c, g);
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v[i][j] *= inv * g[j];
+                store8(dst + c, v[i]);
+            }
+        }
+    } else {
+        for (int c = tid; c < a.D; c += 256) {
+            const float v = (float)src[c] * a.scale + (float)big[c];
+            dst[c] = v;
+            ss += v * v;
+        }
+        const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+        for (int c = tid; c < a.D; c += 256) dst[c] *= inv * w[c];
+    }
+}
+
+template <typename T>
+static void launch_embed_bigram(const BigramArgs& a, const void* table, const void* bigram, const float* w, float* out,
+                                int T_, hipStream_t s) {
+    const int vpt = a.D % 8 ? 0 : ceil_div(a.D / 8, 256);
+#define EB(V) embed_bigram_kernel<T, V><<<T_, 256, 0, s>>>(a, (const T*)table, (const T*)bigram, w, out)
+    if (vpt == 0 || vpt > 4) EB(0);
+    else if (vpt == 1) EB(1);
+    else if (vpt == 2) EB(2);
+    else EB(4);
+#undef EB
+}
+
+// table [V][D], bigram [buckets + 1][D] bf16 or fp32 (f32); last [slots]; cu null: one row per segment
+MRSUM_API int mrsum_embed_bigram(const int* ids, const void* table, const void* bigram, int f32, const float* w,
+                                 const int* cu, const int* row_seg, const int* slots, const int* pos0, int* last,
+                                 float* out, int T, int D, int V, int buckets, int mul_prev, int mul_cur, float scale,
+                                 float eps, hipStream_t s) {
+    if (T <= 0) return 0;
+    if (buckets <= 0 || D <= 0 || V <= 0 || (cu && !row_seg)) return (int)hipErrorInvalidValue;
+    const BigramArgs a{ids, SegArgs{cu, row_seg, slots, pos0}, last, D, V, buckets, mul_prev, mul_cur, scale, eps};
+    if (f32) launch_embed_bigram<float>(a, table, bigram, w, out, T, s);
+    else launch_embed_bigram<bf16>(a, table, bigram, w, out, T, s);
+    return (int)hipGetLastError();
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void gelu_cols_kernel(ProjSrc src, int at, int n, T* __restrict__ out, int ldo) {
+    const int t = blockIdx.y, c = 8 * (blockIdx.x * 256 + threadIdx.x);
+    if (c >= n) return;
+    float v[8];
+    proj8<true>(src, t, at + c, v);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = gelu_tanh<T>(v[j]);
+    store8(out + (size_t)t * ldo + c, v);
+}
+
+// columns [at, at + n) of fp32 slabs [S][T][ld] -> out rows of stride ldo (bf16, or fp32 with out32)
+MRSUM_API int mrsum_gelu_cols(const float* src, int S, int ld, int T, int at, int n, void* out, int out32, int ldo,
+                              hipStream_t s) {
+    if (T <= 0 || n <= 0) return 0;
+    if (S < 1 || at % 8 || n % 8 || ld % 8 || ldo % 8 || at + n > ld || T > 65535) return (int)hipErrorInvalidValue;
+    const ProjSrc p{src, S, (size_t)T * ld, ld};
+    const dim3 g(ceil_div(n / 8, 256), T);
+    if (out32) gelu_cols_kernel<float><<<g, 256, 0, s>>>(p, at, n, (float*)out, ldo);
+    else gelu_cols_kernel<bf16><<<g, 256, 0, s>>>(p, at, n, (bf16*)out, ldo);
     return (int)hipGetLastError();
 }

@@ -1,7 +1,8 @@
 // Row attention over the paged cache for any head width and value width, in bf16 or fp32 storage with fp32
 // arithmetic throughout: one wave per (row, query head).  Every lane scores one key of a 64-key page; the softmax is
 // online across pages; the value sum runs with the lanes over the value columns.  It serves fp32 models and heads
-// the MFMA kernels do not take (attn_prefill.hip / attn_decode.hip), prompt portions and decoded tokens alike.
+// the MFMA kernels do not take (attn_prefill.hip / attn_decode.hip / latent_attn.hip), prompt portions and decoded
+// tokens alike; latent attention runs it with the cached rows as keys and their first columns as values.
 #include "common.h"
 
 constexpr int ROW_PAGE = 64;
@@ -19,7 +20,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const T* __restrict__ q,
                                                         const T* __restrict__ vc, const int* __restrict__ positions,
                                                         const int* __restrict__ seq_idx,
                                                         const int* __restrict__ block_tables, int bt_stride, int H,
-                                                        int G, int dk, int dv, int pitch, float scale,
+                                                        int G, int dk, int dv, int ldv, int pitch, float scale,
                                                         const float* __restrict__ gate, T* __restrict__ out,
                                                         int out_stride) {
     extern __shared__ float sm[];  // per wave: q [dk], p [64]
@@ -61,13 +62,13 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const T* __restrict__ q,
             const int d = lane + 64 * j;
             if (d < dv) {
                 float a = acc[j] * alpha;
-                const T* vr = vc + slab * dv + d;
-                for (int i = 0; i < n; ++i) a += sp[i] * (float)vr[(size_t)i * dv];
+                const T* vr = vc + slab * ldv + d;
+                for (int i = 0; i < n; ++i) a += sp[i] * (float)vr[(size_t)i * ldv];
                 acc[j] = a;
             }
         }
     }
-    const float f = gate[(size_t)t * H + h] / l;
+    const float f = (gate ? gate[(size_t)t * H + h] : 1.f) / l;
     T* o = out + (size_t)t * out_stride + (size_t)h * pitch;
 #pragma unroll
     for (int j = 0; j < ROW_MAXV; ++j) {
@@ -76,23 +77,24 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const T* __restrict__ q,
     }
 }
 
-// q [T][H][dk], caches [pages][G][64][dk | dv], out rows: head h at columns [h * pitch, (h + 1) * pitch), pitch <= dv.
+// q [T][H][dk], caches [pages][G][64][dk | ldv] (values: the first dv columns of a row; the value rows may be the key
+// rows), out rows: head h at columns [h * pitch, (h + 1) * pitch), pitch <= dv.  gate null: ones.
 MRSUM_API int mrsum_attn_rows(const void* q, const void* kc, const void* vc, const int* positions, const int* seq_idx,
-                              const int* block_tables, int bt_stride, int T, int H, int G, int dk, int dv,
+                              const int* block_tables, int bt_stride, int T, int H, int G, int dk, int dv, int ldv,
                               int pitch, float scale, const float* gate, void* out, int out_stride, int f32,
                               hipStream_t s) {
     if (T <= 0) return 0;
-    if (H % G || dk % 4 || pitch > dv || dv > 64 * ROW_MAXV) return (int)hipErrorInvalidValue;
+    if (H % G || dk % 4 || pitch > dv || dv > 64 * ROW_MAXV || ldv < dv) return (int)hipErrorInvalidValue;
     const dim3 grid(T, ceil_div(H, 4));
     const size_t lds = 4 * (dk + ROW_PAGE) * sizeof(float);
     if (lds > 64 * 1024) return (int)hipErrorInvalidValue;
     if (f32)
         attn_rows_kernel<<<grid, 256, lds, s>>>((const float*)q, (const float*)kc, (const float*)vc, positions, seq_idx,
-                                                block_tables, bt_stride, H, G, dk, dv, pitch, scale, gate,
+                                                block_tables, bt_stride, H, G, dk, dv, ldv, pitch, scale, gate,
                                                 (float*)out, out_stride);
     else
         attn_rows_kernel<<<grid, 256, lds, s>>>((const bf16*)q, (const bf16*)kc, (const bf16*)vc, positions, seq_idx,
-                                                block_tables, bt_stride, H, G, dk, dv, pitch, scale, gate,
+                                                block_tables, bt_stride, H, G, dk, dv, ldv, pitch, scale, gate,
                                                 (bf16*)out, out_stride);
     return (int)hipGetLastError();
 }

@@ -168,10 +168,22 @@ __device__ __forceinline__ float4 proj4(const ProjSrc& s, int row, int col) {
     }
 }
 
+// A batch as segments, one per sequence: segment i covers rows [cu[i], cu[i + 1]) (cu null: row i) and continues state
+// slot slots[i] at absolute position pos0[i].
+struct SegArgs {
+    const int* cu;       // [n + 1] or null (one row per segment)
+    const int* row_seg;  // [T] segment of every row (cu given)
+    const int* slots;
+    const int* pos0;
+};
+
 __device__ __forceinline__ void load8(const float* p, float* f) {
     const float4 a = reinterpret_cast<const float4*>(p)[0], b = reinterpret_cast<const float4*>(p)[1];
     f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
 }
+
+__device__ __forceinline__ void ld8(const float* p, float* f) { load8(p, f); }
+__device__ __forceinline__ void ld8(const bf16* p, float* f) { unpack8(*reinterpret_cast<const uint4*>(p), f); }
 
 // 8 / 4 values to bf16 or fp32 storage (aligned)
 __device__ __forceinline__ void store8(bf16* p, const float* f) { *reinterpret_cast<uint4*>(p) = pack8(f); }
@@ -192,5 +204,11 @@ __device__ __forceinline__ float logistic_for(float x) {
     else return logistic(x);
 }
 __device__ __forceinline__ float softplus(float x) { return x > 30.f ? x : log1pf(expf(x)); }
+
+// tanh form of gelu: z times the logistic of 2 sqrt(2 / pi) (z + 0.044715 z^3)
+template <typename T>
+__device__ __forceinline__ float gelu_tanh(float z) {
+    return z * logistic_for<T>(1.5957691216057308f * (z + 0.044715f * z * z * z));
+}
 
 static inline int ceil_div(int a, int b) { return (a + b - 1) / b; }

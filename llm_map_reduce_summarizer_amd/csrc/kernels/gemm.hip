@@ -52,7 +52,7 @@ constexpr int HALF = 16384;
 constexpr int TILE = 4 * HALF;
 constexpr int LOOK = 6;
 
-enum { GEPI_BF16 = 0, GEPI_SWIGLU = 1 };
+enum { GEPI_BF16 = 0, GEPI_SWIGLU = 1, GEPI_GELU = 2 };
 
 typedef int i32x8 __attribute__((ext_vector_type(8)));
 
@@ -318,7 +318,11 @@ __global__ __launch_bounds__(512, 1) void gemm_kernel(const GemmArgs a) {
     };
     // 4 bf16 outputs of tile row rl at byte cbyte of the output tile row; gcol = first weight column of
     // the 16-column group they come from (N % 16 == 0, so the group is wholly in or out of range)
-    auto store4 = [&](int rl, int cbyte, const f32x4& v, int gcol) {
+    auto store4 = [&](int rl, int cbyte, f32x4 v, int gcol) {
+        if constexpr (EPI == GEPI_GELU) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = gelu_tanh<bf16>(v[j]);
+        }
         const uint2 pk = make_uint2(pack2(v[0], v[1]), pack2(v[2], v[3]));
         if constexpr (LEPI) {
             *reinterpret_cast<uint2*>(lds + rl * RB + (((cbyte >> 4) ^ (rl & 7)) << 4) + (cbyte & 15)) = pk;
@@ -432,7 +436,7 @@ MRSUM_API int mrsum_gemm_stamps(unsigned long long* host, int max_words) {
 #endif
 
 // x [M, K] (row stride ldx elements), w [N, K] (ldw), c [M, N] bf16 (ldc) -- or [M, N / 2] for
-// epi 1 (SwiGLU of the [8 gate | 8 up]-interleaved gate_up rows).  fp8: x, w are e4m3fn bytes,
+// epi 1 (SwiGLU of the [8 gate | 8 up]-interleaved gate_up rows) -- or gelu(C) for epi 2 (bf16 only).  fp8: x, w are e4m3fn bytes,
 // sx [M] / sw [N] fp32 row scales; split: x is two-term [hi | lo] of 2K bytes per row over w's K.
 // Requirements (checked by the Python wrapper too): K % 64 (bf16) / K % 128 (fp8), N % 16, 16-byte
 // aligned rows.
@@ -443,6 +447,8 @@ MRSUM_API int mrsum_gemm(const void* x, int ldx, const void* w, int ldw, void* c
     const int es = fp8 ? 1 : 2;
     if ((K * es) % 128 || N % 16 || (ldx * es) % 16 || (ldw * es) % 16 || ldc % 4) return (int)hipErrorInvalidValue;
     if ((size_t)256 * ldx * es >= (1u << 31) || (size_t)256 * ldw * es >= (1u << 31)) return (int)hipErrorInvalidValue;
+    if (epi < GEPI_BF16 || epi > GEPI_GELU || (epi == GEPI_GELU && (fp8 || ((group_m >> 8) & 1))))
+        return (int)hipErrorInvalidValue;
     if (fp8 && (!sx || !sw)) return (int)hipErrorInvalidValue;
     GemmArgs a;
     a.x = (const char*)x; a.w = (const char*)w; a.c = c; a.sx = sx; a.sw = sw;
@@ -489,7 +495,14 @@ MRSUM_API int mrsum_gemm(const void* x, int ldx, const void* w, int ldw, void* c
     if (fp8) {
         if (epi == GEPI_SWIGLU) { GEMM_LAUNCH(true, GEPI_SWIGLU) } else { GEMM_LAUNCH(true, GEPI_BF16) }
     } else {
-        if (epi == GEPI_SWIGLU) { GEMM_LAUNCH(false, GEPI_SWIGLU) } else { GEMM_LAUNCH(false, GEPI_BF16) }
+        if (epi == GEPI_SWIGLU) {
+            GEMM_LAUNCH(false, GEPI_SWIGLU)
+        } else if (epi == GEPI_GELU) {
+            if (lepi) gemm_kernel<false, GEPI_GELU, 8, true, false><<<grid, block, 0, s>>>(a);
+            else gemm_kernel<false, GEPI_GELU, 8, false, false><<<grid, block, 0, s>>>(a);
+        } else {
+            GEMM_LAUNCH(false, GEPI_BF16)
+        }
     }
 #undef GEMM_LAUNCH
     return (int)hipGetLastError();

@@ -11,13 +11,6 @@
 // State S^T is [slots][heads][vdim][N4] fp32 (N4: state size rounded up to 4, zeros past it).
 #include "common.h"
 
-struct SegArgs {
-    const int* cu;       // [n + 1] or null (one row per segment)
-    const int* row_seg;  // [T] segment of every row (cu given)
-    const int* slots;
-    const int* pos0;
-};
-
 // ------------------------------------------------------------------------------------------------ short convolution
 template <bool PARTS, typename T>
 __device__ __forceinline__ void conv_in8(const ProjSrc& src, int row, int col, float* f) {
@@ -355,11 +348,13 @@ __device__ __forceinline__ float4 gated4(const float* y, const float4& z) {
 
 // L lanes per norm group, VPT float4 each in registers (VPT = 0: any part size, re-read for the second pass).  L = 64:
 // a wave per group, four groups per block; L = 256 / 1024: one block per group (few rows: all loads in flight).
-template <bool PARTS, typename TO, int L, int VPT>
+// POST: the norm first, then the gate, and one weight vector shared by the groups (heads).  Columns from col + n to
+// zero_to are zeroed.
+template <bool PARTS, typename TO, int L, int VPT, bool POST>
 __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const float* __restrict__ y, ProjSrc u, int z_at,
                                                                        const float* __restrict__ w, int n, int groups,
                                                                        float eps, float out_scale, TO* __restrict__ out,
-                                                                       int ldo, int col) {
+                                                                       int ldo, int col, int zero_to) {
     __shared__ float red[16];
     constexpr int GPB = L == 64 ? 4 : 1;
     const int gb = (groups + GPB - 1) / GPB;
@@ -368,7 +363,7 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
     const int ng = n / groups;
     const float* yr = y + (size_t)t * n + g * ng;
     const int zc = z_at + g * ng;
-    const float* wr = w + g * ng;
+    const float* wr = POST ? w : w + g * ng;
     TO* o = out + (size_t)t * ldo + col + g * ng;
     const bool on = g < groups;
     float ss = 0.f;
@@ -378,7 +373,8 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
         for (int i = 0; i < VPT; ++i) {
             const int c = 4 * (l + L * i);
             v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (on && c < ng) v[i] = gated4<TO>(yr + c, proj4<PARTS>(u, t, zc + c));
+            if (on && c < ng)
+                v[i] = POST ? *reinterpret_cast<const float4*>(yr + c) : gated4<TO>(yr + c, proj4<PARTS>(u, t, zc + c));
             ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
         }
         ss = L == 64 ? wave_sum(ss) : block_sum(ss, red);
@@ -387,13 +383,18 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
         for (int i = 0; i < VPT; ++i) {
             const int c = 4 * (l + L * i);
             if (on && c < ng) {
-                const float4 k = *reinterpret_cast<const float4*>(wr + c);
+                float4 k = *reinterpret_cast<const float4*>(wr + c);
+                if constexpr (POST) {
+                    const float4 z = proj4<PARTS>(u, t, zc + c);
+                    k.x *= z.x * logistic_for<TO>(z.x); k.y *= z.y * logistic_for<TO>(z.y);
+                    k.z *= z.z * logistic_for<TO>(z.z); k.w *= z.w * logistic_for<TO>(z.w);
+                }
                 store4(o + c, make_float4(v[i].x * inv * k.x, v[i].y * inv * k.y, v[i].z * inv * k.z, v[i].w * inv * k.w));
             }
         }
     } else {
         for (int c = l; on && c < ng; c += L) {
-            const float z = proj_at<PARTS>(u, t, zc + c), v = yr[c] * z * logistic(z);
+            const float z = POST ? 0.f : proj_at<PARTS>(u, t, zc + c), v = POST ? yr[c] : yr[c] * z * logistic(z);
             ss += v * v;
         }
         ss = L == 64 ? wave_sum(ss) : block_sum(ss, red);
@@ -404,24 +405,18 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
         }
     }
     if (g0 == 0)
-        for (int c = col + n + threadIdx.x; c < ldo; c += blockDim.x) out[(size_t)t * ldo + c] = (TO)0.f;
+        for (int c = col + n + threadIdx.x; c < zero_to; c += blockDim.x) out[(size_t)t * ldo + c] = (TO)0.f;
 }
 
-// out[t, col : col + n] of rows [T][ldo]; columns past it are zeroed
-MRSUM_API int mrsum_gated_norm(const float* y, const void* u, int S, int ld, int T, int z_at, const float* w, int n,
-                               int groups, float eps, float out_scale, void* out, int out32, int ldo, int col,
-                               hipStream_t s) {
-    if (T <= 0) return 0;
-    if (groups <= 0 || n % groups || z_at % 8 || ld % 8 || z_at + n > ld || col % 8 || col + n > ldo || ldo % 8 ||
-        (out32 && S < 1))
-        return (int)hipErrorInvalidValue;
-    const ProjSrc p{u, S, (size_t)T * ld, ld};
+template <bool POST>
+static int launch_gated_norm(const float* y, const ProjSrc& p, int T, int z_at, const float* w, int n, int groups, float eps,
+                             float out_scale, void* out, int out32, int ldo, int col, int zero_to, hipStream_t s) {
     const int ng = n / groups, q = ng % 4 ? 0 : ng / 4;  // float4 per part (0: unaligned parts)
     const long long gb = groups, gw = (groups + 3) / 4;
     if ((long long)T * groups > 0x7fffffff) return (int)hipErrorInvalidValue;
 #define GN(PT, TO, L_, V, NB_) \
-    gated_norm_kernel<PT, TO, L_, V><<<(int)((long long)T * (NB_)), L_ == 64 ? 256 : L_, 0, s>>>(                        \
-        y, p, z_at, w, n, groups, eps, out_scale, (TO*)out, ldo, col)
+    gated_norm_kernel<PT, TO, L_, V, POST><<<(int)((long long)T * (NB_)), L_ == 64 ? 256 : L_, 0, s>>>(                  \
+        y, p, z_at, w, n, groups, eps, out_scale, (TO*)out, ldo, col, zero_to)
 #define GN_L(PT, TO)                                        \
     if (!q || q > 4096) GN(PT, TO, 256, 0, gb);             \
     else if (q <= 64 && T > 512) GN(PT, TO, 64, 1, gw);     \
@@ -431,9 +426,22 @@ MRSUM_API int mrsum_gated_norm(const float* y, const void* u, int S, int ld, int
     else if (q <= 1024) GN(PT, TO, 1024, 1, gb);            \
     else GN(PT, TO, 1024, 4, gb);
     if (out32) { GN_L(true, float) }
-    else if (S) { GN_L(true, bf16) }
+    else if (p.S) { GN_L(true, bf16) }
     else { GN_L(false, bf16) }
 #undef GN_L
 #undef GN
     return (int)hipGetLastError();
+}
+
+// out[t, col : col + n] of rows [T][ldo]; columns past it, up to zero_to, are zeroed.  post: norm, then gate; w [n / groups]
+MRSUM_API int mrsum_gated_norm(const float* y, const void* u, int S, int ld, int T, int z_at, const float* w, int n,
+                               int groups, float eps, float out_scale, void* out, int out32, int ldo, int col, int zero_to,
+                               int post, int rows, hipStream_t s) {
+    if (T <= 0) return 0;
+    if (groups <= 0 || n % groups || z_at % 8 || ld % 8 || z_at + n > ld || col % 8 || col + n > ldo || ldo % 8 ||
+        zero_to > ldo || rows < T || (out32 && S < 1))
+        return (int)hipErrorInvalidValue;
+    const ProjSrc p{u, S, (size_t)rows * ld, ld};  // slabs of ``rows`` rows, of which u points at the first used
+    if (post) return launch_gated_norm<true>(y, p, T, z_at, w, n, groups, eps, out_scale, out, out32, ldo, col, zero_to, s);
+    return launch_gated_norm<false>(y, p, T, z_at, w, n, groups, eps, out_scale, out, out32, ldo, col, zero_to, s);
 }

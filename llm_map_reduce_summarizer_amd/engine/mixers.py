@@ -300,6 +300,8 @@ class DeltaMixer(Mixer):
         super().__init__()
         self.spec, self.dtype = spec, dtype
         self.width = up(spec.inner, 16)
+        if device.type == "cuda" and not ops.delta_ok(spec.vdim, spec.dim):
+            raise ValueError("delta heads of %d x %d are wider than the kernels take" % (spec.dim, spec.vdim))
 
     def columns(self, take) -> None:
         s = self.spec

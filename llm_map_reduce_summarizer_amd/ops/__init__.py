@@ -419,6 +419,11 @@ def latent_prefill(q, kv, lat, ctx, m, cu, lens, items, scale, out, col):
 
 
 # ---------------------------------------------------------------- gated delta rule (``m``: engine.mixers.DeltaMixer)
+def delta_ok(vdim, dim):
+    from .hip import delta_step_ok
+    return delta_step_ok(vdim, dim)
+
+
 def delta_mix(x, u, m, a_neg, dt_bias, norm, eps, state, segs, a):
     return _impl(x).delta_mix(x, u, m, a_neg, dt_bias, norm, eps, state, segs, a)
 

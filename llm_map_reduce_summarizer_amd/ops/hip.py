@@ -64,7 +64,7 @@ _SIGS = {
     "mrsum_add_norm32": [_vp, _vp, _c_int, _c_int, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_float, _vp],
     "mrsum_qkv_prep": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp] + [_c_int] * 10 +
                       [_vp, _vp, _vp, _c_float, _c_float, _c_float, _c_float, _vp, _vp, _vp, _c_int, _c_int, _vp],
-    "mrsum_attn_rows": [_vp, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
+    "mrsum_attn_rows": [_vp, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
                         _vp, _vp, _c_int, _c_int, _vp],
     "mrsum_gemm32": [_vp, _c_int, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp],
     "mrsum_conv_silu": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int,
@@ -74,7 +74,18 @@ _SIGS = {
     "mrsum_ssm_chunk": [_vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _vp,
                         _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _vp],
     "mrsum_gated_norm": [_vp, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_float, _c_float, _vp,
-                         _c_int, _c_int, _c_int, _vp],
+                         _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp],
+    "mrsum_embed_bigram": [_vp, _vp, _vp, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int,
+                           _c_int, _c_int, _c_float, _c_float, _vp],
+    "mrsum_gelu_cols": [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _vp],
+    "mrsum_latent_prep": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _vp] + [_c_int] * 8 +
+                         [_vp, _vp, _c_float, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp],
+    "mrsum_head_product": [_vp] + [_c_int] * 6 + [_vp, _c_int, _c_int, _vp] + [_c_int] * 8 + [_vp, _vp, _vp, _vp, _c_int, _vp],
+    "mrsum_latent_rope": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp],
+    "mrsum_latent_gather": [_vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _vp, _vp],
+    "mrsum_delta_step": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp,
+                         _vp, _c_float, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int,
+                         _c_int, _c_int, _vp],
 }
 
 _fns = {}
@@ -647,7 +658,7 @@ def sample_tp(logits: torch.Tensor, st, tok_offset: int, max_reduce) -> None:
 
 # ------------------------------------------------------------------ large-M GEMM (prefill, M > 64)
 GEMM_GROUP_M = 4  # tile rows per raster group (4 x 8 tiles per XCD at a time; 8 measured equal)
-GEMM_EPI_BF16, GEMM_EPI_SWIGLU = 0, 1
+GEMM_EPI_BF16, GEMM_EPI_SWIGLU, GEMM_EPI_GELU = 0, 1, 2
 # group_m bit 8: 32x32-MFMA tiles.  Taken by the fp8 gate_up + SwiGLU GEMM only: +1.7..3.8 % at M = 4k-32k on
 # the 70B shape on two boxes; the 70B fp8 qkv / o / down and every bf16 projection are equal or slower
 # (profiles/r3_gemm_mfma32_experiment.jsonl, r3_gemm_mfma32_fp8_70b.jsonl)
@@ -665,9 +676,9 @@ def _gemm(xp, ldx, wp, ldw, out, M, N, K, fp8, epi, sx, sw, group_m, split=0, gl
 
 
 def gemm(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None, swiglu: bool = False,
-         group_m: Optional[int] = None, glu=None) -> torch.Tensor:
+         group_m: Optional[int] = None, glu=None, gelu: bool = False) -> torch.Tensor:
     """x [M, K] @ w [N, K]^T in bf16 on the 256 x 256-tile MFMA kernel (csrc/kernels/gemm.hip), any M.
-    ``swiglu``: w is the [8 gate | 8 up]-interleaved gate_up weight and the result is silu(gate) * up
+    ``gelu``: the tanh form of gelu of the product.  ``swiglu``: w is the [8 gate | 8 up]-interleaved gate_up weight and the result is silu(gate) * up
     [M, N / 2] (``glu`` = (limit, alpha, shift): the clamped form)."""
     _bf16_cuda(x, w)
     _rows_ok(x)
@@ -684,7 +695,7 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None, s
     if M == 0:
         return out
     return _gemm(_p(x), x.stride(0), _p(w), w.stride(0), out, M, N, K, 0,
-                 GEMM_EPI_SWIGLU if swiglu else GEMM_EPI_BF16, None, None, group_m, glu=glu)
+                 GEMM_EPI_SWIGLU if swiglu else (GEMM_EPI_GELU if gelu else GEMM_EPI_BF16), None, None, group_m, glu=glu)
 
 
 # One backend per op: every bf16 prefill product runs on gemm.hip.  The round-4 experiments that lived here
@@ -1598,7 +1609,7 @@ def attn_rows(q, kcache, vcache, positions, seq_idx, block_tables, hq: int, hkv:
     _req(positions.numel() >= T and seq_idx.numel() >= T, "attn_rows: tables")
     _req(out.dtype == dt and out.stride(1) == 1 and out.shape[0] == T and out.shape[1] >= hq * pitch, "attn_rows: out")
     _check(_fn("mrsum_attn_rows")(_p(q), _p(kcache), _p(vcache), _p(positions), _p(seq_idx), _p(block_tables),
-                                  block_tables.stride(0), T, hq, hkv, dk, dv, pitch, scale, _p(gate), _p(out),
+                                  block_tables.stride(0), T, hq, hkv, dk, dv, dv, pitch, scale, _p(gate), _p(out),
                                   out.stride(0), 1 if dt == torch.float32 else 0, _stream()), "attn_rows")
 
 
@@ -1692,4 +1703,181 @@ def gated_norm(y, u, z_at: int, w, norm_groups: int, eps: float, out_scale: floa
          and out.shape[0] == T and col % 8 == 0 and col + n <= out.shape[1] and out.shape[1] % 8 == 0,
          "gated_norm: shapes")
     _check(_fn("mrsum_gated_norm")(_p(y), ptr, S, ld, T, z_at, _p(w), n, norm_groups, eps, out_scale, _p(out),
-                                   1 if out.dtype == torch.float32 else 0, out.shape[1], col, _stream()), "gated_norm")
+                                   1 if out.dtype == torch.float32 else 0, out.shape[1], col, out.shape[1], 0, T,
+                                   _stream()), "gated_norm")
+
+
+# ------------------------------------------------------------------ bigram embedding, plain gelu feed-forward
+def embed_bigram(ids, segs, table, bigram, scale: float, mul_prev: int, mul_cur: int, w, eps: float, last) -> torch.Tensor:
+    T = ids.numel()
+    _i32(ids, last)
+    _f32(w)
+    V, D = table.shape
+    _req(table.is_cuda and table.is_contiguous() and bigram.is_contiguous() and bigram.dtype == table.dtype
+         and table.dtype in (torch.bfloat16, torch.float32) and bigram.shape[1] == D and bigram.shape[0] >= 2
+         and w.numel() == D, "embed_bigram: tables")
+    cu, row_seg = _seg_ptrs(segs, T, "embed_bigram")
+    out = torch.empty(T, D, dtype=torch.float32, device=table.device)
+    _check(_fn("mrsum_embed_bigram")(_p(ids), _p(table), _p(bigram), 1 if table.dtype == torch.float32 else 0, _p(w), cu,
+                                     row_seg, _p(segs.slots), _p(segs.pos0), _p(last), _p(out), T, D, V,
+                                     bigram.shape[0] - 1, mul_prev, mul_cur, scale, eps, _stream()), "embed_bigram")
+    return out
+
+
+def gelu_cols(u, at: int, n: int, out, col: int) -> None:
+    """out[:, col : col + n] = gelu of columns [at, at + n) of fp32 slabs ``u``."""
+    ptr, S, ld, T = _src(u, torch.bfloat16, "gelu_cols")
+    _req(S >= 1 and at + n <= ld and out.stride(1) == 1 and out.shape[0] == T and col % 8 == 0 and col + n <= out.shape[1]
+         and out.stride(0) % 8 == 0 and out.dtype in (torch.bfloat16, torch.float32), "gelu_cols: shapes")
+    es = out.element_size()
+    _check(_fn("mrsum_gelu_cols")(ptr, S, ld, T, at, n, out.data_ptr() + es * col, 1 if es == 4 else 0, out.stride(0),
+                                  _stream()), "gelu_cols")
+
+
+def project_gelu(x, w, n: int, out, col: int, cols: int):
+    """Decode row counts and 32-bit mode: one product of all rows of ``w`` whose gelu columns are summed from its slabs.
+    More rows: two MFMA GEMMs, the second with the gelu in its epilogue, straight into ``out``."""
+    M = x.shape[0]
+    _req(n % 8 == 0 and n + cols <= w.shape[0], "project_gelu: rows")
+    if x.dtype == torch.bfloat16 and M > STREAM_MAX_M:
+        gemm(x, w[n: n + cols], out=out[:, col: col + cols], gelu=True)
+        return gemm(x, w[:n])
+    from . import project
+    u = project(x, w, "qkv")
+    if u.dim() == 2:  # a shape only the GEMM takes
+        gemm(x, w[n: n + cols], out=out[:, col: col + cols], gelu=True)
+    else:
+        gelu_cols(u, n, cols, out, col)
+    return u
+
+
+# ------------------------------------------------------------------ latent attention (``m``: engine.mixers.LatentMixer)
+def latent_prefill_form(qw: int, vp: int):
+    """(key width, value width, query rows per workgroup) of the prompt-portion kernel that takes heads of ``qw`` key and
+    ``vp`` value columns, or None."""
+    return None
+
+
+def latent_decode_form(rank: int, row: int):
+    return None
+
+
+def _rotary_ok(cs, rot: int, positions, n: int, what: str) -> None:
+    _i32(positions)
+    _req(cs.is_cuda and cs.dtype == torch.float32 and cs.is_contiguous() and cs.shape[1:] == (rot // 2, 2)
+         and positions.numel() >= n, what + ": rotation table / positions")
+
+
+def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, block_tables, cache, page: int, dtype):
+    sp = m.spec
+    ptr, S, ld, T = _src(u, dtype, "latent_prep")
+    _i32(seq_idx, block_tables)
+    _f32(dq_norm)
+    _rotary_ok(cs, sp.rot_dim, positions, T, "latent_prep")
+    own = dkv_norm is not None
+    _req(dq_norm.numel() == sp.q_rank and m.dq + sp.q_rank <= ld and seq_idx.numel() >= T and block_tables.dim() == 2,
+         "latent_prep: shapes")
+    if own:
+        _f32(dkv_norm)
+        _req(dkv_norm.numel() == sp.kv_rank and m.dkv + sp.kv_rank <= ld and m.dkr + sp.rot_dim <= ld, "latent_prep: latents")
+        _row_cache(cache, 1, page, m.row, dtype, "latent_prep")
+    out = torch.empty(T, m.cq, dtype=dtype, device=u.device)
+    _check(_fn("mrsum_latent_prep")(ptr, S, ld, T, 1 if dtype == torch.float32 else 0, _p(out), m.cq,
+                                    _p(cache) if own else None, m.dq, sp.q_rank, m.dkv if own else -1, sp.kv_rank,
+                                    m.dkr if own else 0, sp.rot_dim, m.rank8, m.row, _p(dq_norm), _p(dkv_norm), eps, _p(cs),
+                                    _p(positions), _p(seq_idx), _p(block_tables), block_tables.stride(0), page,
+                                    _stream()), "latent_prep")
+    return out
+
+
+def _head_product(x, S, ldx, xrows, rows, xs, xk, w, out, os, H, rot=(0, 0, 0, 0), cs=None, positions=None, parts=None):
+    _, N, K = w.shape
+    _req(w.is_cuda and w.is_contiguous() and w.shape[0] == H and w.dtype == out.dtype and out.stride(1) == 1
+         and (H - 1) * os + N <= out.shape[1] and rows <= out.shape[0] and out.data_ptr() % 16 == 0, "head_product: operands")
+    po, ml, splits = parts if parts is not None else (None, None, 0)
+    _check(_fn("mrsum_head_product")(x, S, ldx, xrows, rows, xs, xk, _p(w), N, K, _p(out),
+                                     1 if out.dtype == torch.float32 else 0, os, out.stride(0), H, *rot, _p(cs),
+                                     _p(positions), _p(po), _p(ml), splits, _stream()), "head_product")
+
+
+def latent_absorb(q, n: int, m, w_uk, cs, positions, dtype) -> torch.Tensor:
+    sp = m.spec
+    ptr, S, ld, T = _src(q, dtype, "latent_absorb")
+    _rotary_ok(cs, sp.rot_dim, positions, n, "latent_absorb")
+    _req(0 < n <= T and sp.heads * m.qw <= ld and tuple(w_uk.shape[:2]) == (sp.heads, m.rank8), "latent_absorb: shapes")
+    out = torch.empty(n, sp.heads * m.row, dtype=dtype, device=q.device)
+    _head_product(ptr, S, ld, T, n, m.qw, m.dim8, w_uk, out, m.row, sp.heads, (sp.rot_dim, m.rot8, m.dim8, m.rank8), cs,
+                  positions)
+    return out
+
+
+def latent_rows(q, cache, positions, seq_idx, block_tables, heads: int, rank: int, page: int, scale: float):
+    T, dt, row = q.shape[0], q.dtype, cache.shape[3]
+    _row_cache(cache, 1, page, row, dt, "latent_rows")
+    _i32(positions, seq_idx, block_tables)
+    _req(dt in (torch.bfloat16, torch.float32) and page == 64 and q.is_contiguous() and q.shape[1] == heads * row
+         and rank <= min(row, 512) and positions.numel() >= T and seq_idx.numel() >= T, "latent_rows: shapes")
+    out = torch.empty(T, heads * rank, dtype=dt, device=q.device)
+    _check(_fn("mrsum_attn_rows")(_p(q), _p(cache), _p(cache), _p(positions), _p(seq_idx), _p(block_tables),
+                                  block_tables.stride(0), T, heads, 1, row, rank, row, rank, scale, None, _p(out),
+                                  out.stride(0), 1 if dt == torch.float32 else 0, _stream()), "latent_rows")
+    return out
+
+
+def latent_out(o, m, w_uv, a, col: int) -> None:
+    H, n = m.spec.heads, o.shape[0]
+    _req(o.is_cuda and o.is_contiguous() and o.shape[1] == H * m.rank8 and o.dtype == a.dtype and n <= a.shape[0]
+         and tuple(w_uv.shape[:2]) == (H, m.vp) and col % 8 == 0, "latent_out: shapes")
+    _head_product(_p(o), 1 if o.dtype == torch.float32 else 0, o.shape[1], n, n, m.rank8, m.rank8, w_uv, a[:, col:], m.vp, H)
+
+
+def latent_rope(q, first: int, m, cs, positions) -> torch.Tensor:
+    sp = m.spec
+    ptr, S, ld, T = _src(q, torch.bfloat16, "latent_rope")
+    _rotary_ok(cs, sp.rot_dim, positions, T, "latent_rope")
+    w = sp.heads * m.qw
+    _req(0 <= first < T and w <= ld, "latent_rope: shapes")
+    out = torch.empty(T - first, w, dtype=torch.bfloat16, device=q.device) if S else q[first:]
+    _check(_fn("mrsum_latent_rope")(ptr, S, ld, T, first, _p(out), out.stride(0), sp.heads, m.qw, m.dim8, sp.rot_dim, _p(cs),
+                                    _p(positions), _stream()), "latent_rope")
+    return out
+
+
+def latent_gather(cache, ctx, block_tables, width: int, page: int) -> torch.Tensor:
+    row = cache.shape[3]
+    _row_cache(cache, 1, page, row, torch.bfloat16, "latent_gather")
+    _i32(block_tables, ctx.pages)
+    _req(page == 64 and width % 8 == 0 and width >= row and block_tables.dim() == 2
+         and all(0 <= s < block_tables.shape[0] and c <= block_tables.shape[1] * 64
+                 for s, c in zip(ctx.slot_host, ctx.ctx)), "latent_gather: tables")
+    out = torch.empty(ctx.rows, width, dtype=torch.bfloat16, device=cache.device)
+    _check(_fn("mrsum_latent_gather")(_p(cache), _p(ctx.pages), ctx.pages.shape[0], _p(block_tables),
+                                      block_tables.stride(0), row, width, _p(out), _stream()), "latent_gather")
+    return out
+
+
+# ------------------------------------------------------------------ gated delta rule (``m``: engine.mixers.DeltaMixer)
+def delta_step_ok(vdim: int, dim: int) -> bool:
+    """Head sizes the stepped kernel holds in registers (delta.hip)."""
+    return dim <= 256 and vdim <= (512 if dim <= 32 else 256 if dim <= 128 else 128)
+
+
+def delta_mix(x, u, m, a_neg, dt_bias, norm, eps: float, state, segs, a) -> None:
+    """Leading one-row segments (decoded tokens) and 32-bit models token by token, with the output norm in the same
+    launch; prompt portions of 16-bit models in chunks on MFMA."""
+    sp = m.spec
+    H, G, P, N = sp.heads, sp.kv_heads, sp.vdim, sp.dim
+    ptr, S, ld, T = _src(u, x.dtype, "delta_mix")
+    _f32(a_neg, dt_bias, norm, state)
+    x32 = x.dtype == torch.float32
+    _req(x.is_cuda and x.is_contiguous() and x.shape[0] == T and x.shape[1] >= m.xv + H * P and a.shape[0] == T
+         and a.dtype == x.dtype and a.stride(1) == 1 and m.col + m.width <= a.shape[1], "delta_mix: rows")
+    _req(a_neg.numel() == dt_bias.numel() == H and norm.numel() == P
+         and tuple(state.shape[1:]) == (H, P, -(-N // 4) * 4), "delta_mix: parameters")
+    _req(max(m.b + H, m.a + H, m.g + H * P) <= ld, "delta_mix: columns")
+    cu, _ = _seg_ptrs(segs, T, "delta_mix")
+    stepped = segs.n
+    if stepped:
+        _check(_fn("mrsum_delta_step")(_p(x), x.shape[1], 1 if x32 else 0, m.xk, m.xv, ptr, S, ld, T, m.b, m.a, m.g,
+                                       _p(dt_bias), _p(a_neg), _p(norm), eps, _p(state), cu, _p(segs.slots), _p(segs.pos0),
+                                       0, stepped, _p(a), a.stride(0), m.col, m.width, H, G, P, N, _stream()), "delta_step")
