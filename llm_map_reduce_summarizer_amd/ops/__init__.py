@@ -352,7 +352,7 @@ def latent_decode_ok(rank8, row):
 def latent_block_rows(qw, vp):
     """Query rows per workgroup of the prompt-portion kernel."""
     from .hip import latent_prefill_form
-    return latent_prefill_form(qw, vp)[2]
+    return latent_prefill_form(qw, vp)[1]
 
 
 def latent_items(lens, rows):

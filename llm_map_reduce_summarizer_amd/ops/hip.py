@@ -83,6 +83,12 @@ _SIGS = {
     "mrsum_head_product": [_vp] + [_c_int] * 6 + [_vp, _c_int, _c_int, _vp] + [_c_int] * 8 + [_vp, _vp, _vp, _vp, _c_int, _vp],
     "mrsum_latent_rope": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp],
     "mrsum_latent_gather": [_vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _vp, _vp],
+    "mrsum_latent_prefill": [_vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _vp, _vp, _vp,
+                             _vp, _c_int, _c_int, _vp, _c_int, _c_float, _c_int, _vp],
+    "mrsum_latent_decode": [_vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _vp, _vp, _vp],
+    "mrsum_delta_chunk": [_vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp,
+                          _vp, _c_int, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp],
+    "mrsum_delta_chunk_pieces": [],
     "mrsum_delta_step": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp,
                          _vp, _c_float, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int,
                          _c_int, _c_int, _vp],
@@ -1752,14 +1758,37 @@ def project_gelu(x, w, n: int, out, col: int, cols: int):
 
 
 # ------------------------------------------------------------------ latent attention (``m``: engine.mixers.LatentMixer)
+# (16-column key steps, key width, value width) of the instantiated prompt-portion kernels (latent_attn.hip)
+LATENT_FORMS = ((4, 64, 64), (8, 128, 128), (12, 192, 128))
+LATENT_BLOCK = 256  # query rows per workgroup
+LATENT_DECODE_FORMS = ((128, 128), (256, 320), (512, 576))  # (latent width, row width)
+
+
 def latent_prefill_form(qw: int, vp: int):
-    """(key width, value width, query rows per workgroup) of the prompt-portion kernel that takes heads of ``qw`` key and
-    ``vp`` value columns, or None."""
-    return None
+    """(form, query rows per workgroup) of the prompt-portion kernel that takes heads of ``qw`` key and ``vp`` value
+    columns, or None."""
+    return next(((f, LATENT_BLOCK) for f, k, v in LATENT_FORMS if qw <= k and vp <= v), None)
 
 
 def latent_decode_form(rank: int, row: int):
-    return None
+    return next(((r, w) for r, w in LATENT_DECODE_FORMS if rank <= r and row <= w), None)
+
+
+def block_items(lens, rows: int) -> torch.Tensor:
+    """(portion, first query row) of every block of ``rows`` query rows, heaviest (latest) blocks first."""
+    items = sorted(((qb, i) for i, n in enumerate(lens) for qb in range(0, int(n), rows)), key=lambda e: -e[0])
+    return torch.tensor([(i, qb) for qb, i in items], dtype=torch.int32).reshape(-1, 2)
+
+
+class LatentWorkspace:
+    """Split-K partial sums of latent_decode for ``B`` rows whose contexts reach ``max_ctx``: as many (sequence, head
+    block, split) workgroups as there are CUs (one fits a CU), at least a page each."""
+
+    def __init__(self, B: int, heads: int, rank: int, max_ctx: int, device):
+        groups = max(1, B * -(-heads // 32))
+        self.splits = max(1, min(N_CU // groups, -(-max_ctx // 64), 256))
+        self.part_o = torch.empty(B * heads * self.splits * rank, dtype=torch.float32, device=device)
+        self.part_ml = torch.empty(B * heads * self.splits * 2, dtype=torch.float32, device=device)
 
 
 def _rotary_ok(cs, rot: int, positions, n: int, what: str) -> None:
@@ -1856,10 +1885,78 @@ def latent_gather(cache, ctx, block_tables, width: int, page: int) -> torch.Tens
     return out
 
 
+def latent_prefill(q, kv, lat, ctx, m, cu, lens, items, scale: float, out, col: int) -> None:
+    sp = m.spec
+    form = latent_prefill_form(m.qw, m.vp)
+    _bf16_cuda(q, kv, lat, out)
+    _rows_ok(q)
+    _i32(cu, items, ctx.prefix, ctx.base)
+    T = sum(lens)
+    _req(form is not None and q.shape[0] == T == out.shape[0] and cu.numel() == len(lens) + 1 == ctx.base.numel()
+         and ctx.prefix.numel() == len(lens) and kv.shape[0] == lat.shape[0] == ctx.rows
+         and all(c == p + n for c, p, n in zip(ctx.ctx, ctx.prefix_host, lens)), "latent_prefill: portions")
+    _req(kv.is_contiguous() and lat.is_contiguous() and out.stride(1) == 1 and out.data_ptr() % 16 == 0 and col % 8 == 0
+         and col + sp.heads * m.vp <= out.shape[1] and items.shape[0] == sum(-(-n // form[1]) for n in lens),
+         "latent_prefill: operands")
+    _check(_fn("mrsum_latent_prefill")(_p(q), q.stride(0), m.qw, _p(kv), kv.shape[1], m.dim8, m.kv_v, m.vp, _p(lat),
+                                       lat.shape[1], m.rank8, _p(cu), _p(ctx.prefix), _p(ctx.base), _p(items),
+                                       items.shape[0], sp.heads, out.data_ptr() + 2 * col, out.stride(0), scale, form[0],
+                                       _stream()), "latent_prefill")
+
+
+def latent_decode(q, cache, block_tables, positions, heads: int, rank: int, page: int, scale: float, ws=None):
+    """(partial sums, (maximum, sum) pairs, splits) of single tokens; head_product merges them."""
+    B, row = q.shape[0], cache.shape[3]
+    _bf16_cuda(q)
+    _row_cache(cache, 1, page, row, torch.bfloat16, "latent_decode")
+    _i32(block_tables, positions)
+    _req(page == 64 and q.is_contiguous() and q.shape[1] == heads * row and latent_decode_form(rank, row) is not None
+         and block_tables.dim() == 2 and block_tables.shape[0] >= B and positions.numel() >= B, "latent_decode: shapes")
+    if ws is None:
+        ws = LatentWorkspace(B, heads, rank, block_tables.shape[1] * page, q.device)
+    _req(ws.part_o.numel() >= B * heads * ws.splits * rank and ws.part_ml.numel() >= 2 * B * heads * ws.splits,
+         "latent_decode: workspace")
+    _check(_fn("mrsum_latent_decode")(_p(q), _p(cache), _p(block_tables), block_tables.stride(0), _p(positions), B, heads,
+                                      rank, row, ws.splits, scale, _p(ws.part_o), _p(ws.part_ml), _stream()),
+           "latent_decode")
+    return ws.part_o, ws.part_ml, ws.splits
+
+
+def latent_out_parts(parts, m, w_uv, a, col: int) -> None:
+    H, n = m.spec.heads, a.shape[0]
+    _req(tuple(w_uv.shape[:2]) == (H, m.vp) and col % 8 == 0 and parts[0].numel() >= n * H * parts[2] * m.rank8,
+         "latent_out_parts: shapes")
+    _head_product(None, -1, 0, n, n, 0, m.rank8, w_uv, a[:, col:], m.vp, H, parts=parts)
+
+
 # ------------------------------------------------------------------ gated delta rule (``m``: engine.mixers.DeltaMixer)
 def delta_step_ok(vdim: int, dim: int) -> bool:
     """Head sizes the stepped kernel holds in registers (delta.hip)."""
     return dim <= 256 and vdim <= (512 if dim <= 32 else 256 if dim <= 128 else 128)
+
+
+def delta_chunk_ok(vdim: int, dim: int) -> bool:
+    """Head sizes the chunked kernels take (delta_chunk.hip)."""
+    return vdim % 8 == 0 and dim % 8 == 0 and dim <= 256
+
+
+def delta_chunks(lens, first: int):
+    """Work lists of the chunked delta rule over segments ``first``.. of row counts ``lens``: (segment, first row, end row,
+    first chunk) per segment and (first row, end row) per 64-token chunk."""
+    segs, chunks, row = [], [], sum(lens[:first])
+    for i in range(first, len(lens)):
+        segs.append((i, row, row + lens[i], len(chunks)))
+        chunks += [(b, min(b + 64, row + lens[i])) for b in range(row, row + lens[i], 64)]
+        row += lens[i]
+    return segs, chunks
+
+
+def delta_waves(vdim: int, dim: int, pairs: int) -> int:
+    """Waves of 16 value columns per workgroup: as many as leave no CU without a workgroup."""
+    for w in (8, 4) if dim <= 128 else (4,):
+        if 16 * (w // 2) < vdim and pairs * -(-vdim // (16 * w)) >= N_CU:
+            return w
+    return 2
 
 
 def delta_mix(x, u, m, a_neg, dt_bias, norm, eps: float, state, segs, a) -> None:
@@ -1877,7 +1974,26 @@ def delta_mix(x, u, m, a_neg, dt_bias, norm, eps: float, state, segs, a) -> None
     _req(max(m.b + H, m.a + H, m.g + H * P) <= ld, "delta_mix: columns")
     cu, _ = _seg_ptrs(segs, T, "delta_mix")
     stepped = segs.n
+    if segs.cu is not None and not x32 and delta_chunk_ok(P, N) and x.shape[1] % 8 == 0:
+        stepped = next((i for i, n in enumerate(segs.lens) if n != 1), segs.n)
     if stepped:
         _check(_fn("mrsum_delta_step")(_p(x), x.shape[1], 1 if x32 else 0, m.xk, m.xv, ptr, S, ld, T, m.b, m.a, m.g,
                                        _p(dt_bias), _p(a_neg), _p(norm), eps, _p(state), cu, _p(segs.slots), _p(segs.pos0),
                                        0, stepped, _p(a), a.stride(0), m.col, m.width, H, G, P, N, _stream()), "delta_step")
+    if stepped < segs.n:
+        y0 = sum(segs.lens[:stepped])
+        if "delta_chunks" not in segs.plans:  # built once per pass, used by every layer
+            dev = lambda v: torch.tensor(v, dtype=torch.int32).to(u.device, non_blocking=True)  # noqa: E731
+            segs.plans["delta_chunks"] = tuple(dev(v) for v in delta_chunks(segs.lens, stepped))
+        runs, chunks = segs.plans["delta_chunks"]
+        nc = chunks.shape[0]
+        frags = torch.empty(nc * H * _fn("mrsum_delta_chunk_pieces")() * 4, dtype=torch.int32, device=u.device)
+        vec = torch.empty(nc * H * 256, dtype=torch.float32, device=u.device)
+        y = torch.empty(T - y0, H * P, dtype=torch.float32, device=u.device)
+        _check(_fn("mrsum_delta_chunk")(_p(x), x.shape[1], m.xk, m.xv, ptr, S, ld, T, m.b, m.a, _p(dt_bias), _p(a_neg),
+                                        _p(state), _p(segs.slots), _p(segs.pos0), _p(runs), runs.shape[0], _p(chunks), nc,
+                                        _p(frags), _p(vec), _p(y), y0, H, G, P, N, delta_waves(P, N, H * runs.shape[0]),
+                                        _stream()), "delta_chunk")
+        rows = a[y0:]
+        _check(_fn("mrsum_gated_norm")(_p(y), ptr + y0 * ld * (4 if S else 2), S, ld, T - y0, m.g, _p(norm), H * P, H, eps,
+                                       1.0, _p(rows), 0, a.stride(0), m.col, m.col + m.width, 1, T, _stream()), "gated_norm")

@@ -98,12 +98,12 @@ def latent_attend(q, lat, kr, w_uk, w_uv, c, planted=()):
     head after the other.  Returns [T, heads * vdim]."""
     T, H, d, dv = q.shape[0], c["heads"], c["dim"], c["vdim"]
     out = torch.zeros(T, H * dv, dtype=F)
+    qr = torch.stack([rotate(q[i, :, d:], i, c["rot"], planted) for i in range(T)])
     for a in range(H):
         k = lat @ w_uk[a * d:(a + 1) * d].T
         v = lat @ w_uv[a * dv:(a + 1) * dv].T
         for i in range(T):
-            qr = rotate(q[i, a, d:], i, c["rot"], planted)
-            s = (k[:i + 1] @ q[i, a, :d] + kr[:i + 1] @ qr) * c["scale"]
+            s = (k[:i + 1] @ q[i, a, :d] + kr[:i + 1] @ qr[i, a]) * c["scale"]
             if "drop_first_key" in planted and i > 0:
                 s[0] = -math.inf
             p = torch.exp(s - s.max())

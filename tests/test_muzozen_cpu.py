@@ -1,0 +1,261 @@
+"""The Muzozen design in the engine against its float64 oracle (tests/muzozen_oracle.py), on the CPU operations: the
+model, its weights, the paged latent cache and recurrent state, portions, batches, reuse and greedy generation.  The GPU
+tests run the same schedules on the HIP kernels."""
+import io
+import json
+import math
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+import muzozen_cases as M
+import muzozen_oracle as O
+from llm_map_reduce_summarizer_amd.engine.engine import SamplingParams
+
+F32 = torch.float32
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+
+@pytest.mark.parametrize("name", sorted(M.CONFIGS))
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_prompt_and_token_by_token(name, dtype, tmp_path):
+    eng = M.engine(name, tmp_path, "cpu", dtype)
+    ids = M.tokens(name, 70)
+    want = M.expected(name, ids)
+    M.check(M.feed(eng, "a", ids, [70]), want, dtype, "one portion")
+    M.check(M.feed(eng, "b", ids, [1] * 70), want, dtype, "token by token")
+    assert eng.kv.alloc.available() == 32 and eng.kv.state.alloc.available() == 4
+
+
+@pytest.mark.parametrize("sizes", [[2], [3, 1, 64], [63, 2], [65], [17, 1, 1, 30]])
+def test_portions(sizes, tmp_path):
+    eng = M.engine("mixed", tmp_path, "cpu", F32)
+    ids = M.tokens("mixed", 140)
+    M.check(M.feed(eng, "a", ids, M.cuts(140, sizes)), M.expected("mixed", ids), F32, str(sizes))
+
+
+def test_unequal_requests_share_batches_and_reuse_slots(tmp_path):
+    """Six requests of unequal length through three slots and a pool that holds three of them at most: portions of some
+    beside single tokens of others; pages, state slots and their last tokens taken over from ended requests."""
+    lengths = {"a": 131, "b": 5, "c": 64, "d": 1, "e": 90, "f": 65}
+    eng = M.engine("mixed", tmp_path, "cpu", F32, max_num_seqs=3, kv_pages=8)
+    reqs = {r: M.tokens("mixed", n, seed=i) for i, (r, n) in enumerate(lengths.items())}
+    got = M.feed_mixed(eng, reqs, M.mixed_plan(lengths, [1, 30, 2, 1, 64, 1], live=3))
+    for r, ids in reqs.items():
+        M.check(got[r], M.expected("mixed", ids), F32, r)
+
+
+def test_request_left_out_of_steps_continues(tmp_path):
+    eng = M.engine("odd", tmp_path, "cpu", F32)
+    a, b = M.tokens("odd", 40, 1), M.tokens("odd", 30, 2)
+    first = eng.step([("a", a[:20], range(20))])[0]
+    M.check(M.feed(eng, "b", b, [7, 1, 22]), M.expected("odd", b), F32)
+    rest = eng.step([("a", a[20:], range(20))], ["a"])[0]
+    M.check(torch.cat([first, rest]), M.expected("odd", a), F32)
+
+
+def test_layer_residuals(tmp_path):
+    eng = M.engine("mixed", tmp_path, "cpu", F32)
+    seen = {}
+    eng.model.layer_hook = lambda i, r: seen.__setitem__(i, r.clone())
+    ids, want = M.tokens("mixed", 20), []
+    O.forward(M.CONFIGS["mixed"], M.weights("mixed"), ids, layers_out=want)
+    M.feed(eng, "a", ids, [20])
+    assert len(seen) == len(want) == 7
+    for i, w in enumerate(want):
+        assert float((seen[i].double() - w).abs().max() / w.abs().max()) < 1e-5, i
+
+
+@pytest.mark.parametrize("planted", ["first_pair_zero", "plain_rotation", "drop_first_key", "read_before_write",
+                                     "state_reset_64"])
+def test_inputs_reveal_planted_mistakes(planted):
+    """A mistake in one mechanism of the oracle moves the logits far beyond what the comparisons allow."""
+    ids = M.tokens("mixed", 140)
+    e = M.error(M.expected("mixed", ids, (planted,)), M.expected("mixed", ids))
+    assert float(e.max()) > 2 * M.TOL[torch.bfloat16], planted
+    if planted == "state_reset_64":
+        assert float(e[:64].max()) < 1e-9 and float(e[64:68].max()) > 100 * M.TOL[F32]
+    if planted == "drop_first_key":
+        assert float(e[0]) < 1e-9
+
+
+def test_rotation_table():
+    """Frequencies and factor of YaRN: kept, ramped and slowed pairs, clamped ends, a ramp of no width, no scaling."""
+    from llm_map_reduce_summarizer_amd.engine.config import RotarySpec, YarnSpec
+    from llm_map_reduce_summarizer_amd.ops.reference import rotary_table, rotate_half
+    cases = [M.rot(24), M.rot(64, base=1e6, factor=40.0, original=4096, fast=32.0, slow=1.0), M.rot(8, base=500.0),
+             M.rot(16, base=100.0, factor=8.0, original=7, fast=1.0, slow=1.0), M.rot(6, factor=None),
+             M.rot(12, factor=1.0, original=100000, fast=100.0, slow=2e-4)]
+    for r in cases:
+        s = r["scaling"]
+        spec = RotarySpec(r["dims"], r["base"], YarnSpec(s["factor"], s["original"], s["fast"], s["slow"]) if s else None)
+        cs = rotary_table(3000, spec)
+        x = torch.randn(r["dims"], generator=torch.Generator().manual_seed(1), dtype=torch.float64)
+        for p in (0, 1, 63, 2999):
+            want = O.rotate(x, p, r)
+            assert float((rotate_half(x, cs[p].double()) - want).abs().max()) < 1e-6, (r, p)
+    assert abs(float(cs[0, 0, 0]) - (0.1 * math.log(1.0) + 1.0)) < 1e-7
+
+
+def test_bigram_rows_follow_the_sequence():
+    """The pair of a portion's first token reaches back into the previous portion; a sequence's first token has its own
+    row; large ids and multipliers do not overflow."""
+    from llm_map_reduce_summarizer_amd import ops
+    D, V, B = 8, 200000, 65537
+    g = torch.Generator().manual_seed(3)
+    table, big, w = torch.randn(V, D, generator=g), torch.randn(B + 1, D, generator=g), torch.ones(D)
+    c = {"scale": 2.0, "bigram": {"buckets": B, "mul_prev": 1000003, "mul_cur": 999983}}
+    ids = torch.randint(0, V, (20,), generator=g).tolist()
+    want = O.embed(ids, {"embed": table.double(), "bigram": big.double(), "embed.norm": w.double()}, c, 1e-6)
+    last, got = torch.full((4,), 77, dtype=torch.int32), []
+    for b, e in ((0, 7), (7, 8), (8, 9), (9, 20)):
+        segs = ops.Segments(torch.tensor([2]), torch.tensor([b]), torch.tensor([0, e - b]), torch.zeros(e - b), [e - b])
+        got.append(ops.embed_bigram(torch.tensor(ids[b:e], dtype=torch.int32), segs, table, big, 2.0, 1000003, 999983, w,
+                                    1e-6, last))
+    assert float((torch.cat(got).double() - want).abs().max()) < 1e-5
+    assert last.tolist() == [77, 77, ids[-1], 77]
+
+
+@pytest.mark.parametrize("kw", [{}, {"prefill_chunk": 64}, {"max_num_seqs": 2, "kv_pages": 9}])
+def test_greedy_generation(kw, tmp_path):
+    """LLMEngine.generate: packed prefill (whole or sliced prompts), continuous batching over fewer slots than requests,
+    decode with compaction, stop by length."""
+    eng = M.engine("mixed", tmp_path, "cpu", F32, **kw)
+    prompts = [M.tokens("mixed", n, seed=n) for n in (3, 130, 64, 1, 77)]
+    outs = eng.generate(prompts, [SamplingParams(n, 0.0, 1) for n in (9, 12, 6, 20, 2)])
+    for p, o in zip(prompts, outs):
+        M.check_greedy("mixed", p, o.token_ids, 1e-4)
+    assert [len(o.token_ids) for o in outs] == [9, 12, 6, 20, 2]
+    assert eng.kv.alloc.available() == eng.kv.num_pages - 1
+    assert eng.kv.state.alloc.available() == eng.max_num_seqs
+
+
+def test_requests_join_a_running_batch(tmp_path):
+    eng = M.engine("mixed", tmp_path, "cpu", F32, prefill_chunk=64, sync_every=2)
+    late = [M.tokens("mixed", n, seed=50 + n) for n in (100, 5)]
+    fed = []
+
+    def feeder(done):
+        if not fed:
+            fed.append(1)
+            return [(p, SamplingParams(7, 0.0, 1)) for p in late]
+        return []
+    first = M.tokens("mixed", 33, seed=9)
+    outs = eng.generate([first], [SamplingParams(25, 0.0, 1)], feeder=feeder)
+    assert eng.stats["interleaved_prefills"] == 2
+    for p, o in zip([first] + late, outs):
+        M.check_greedy("mixed", p, o.token_ids, 1e-4)
+
+
+def test_cache_holds_one_row_per_token_of_own_layers(tmp_path):
+    eng = M.engine("mixed", tmp_path, "cpu", F32)
+    assert [None if k is None else tuple(k.shape[1:]) for k in eng.kv.k] == [
+        (1, 64, 72), None, None, (1, 64, 96), None, None, None]
+    assert eng.cfg.kv_bytes_per_token(4) == 4 * (48 + 24 + 88 + 8)
+    assert [s is not None for s in eng.model.state_shapes()] == [False, True, False, False, True, False, False]
+
+
+def test_configuration_and_checkpoint_errors(tmp_path):
+    from llm_map_reduce_summarizer_amd.engine.config import HybridConfig, get_model_config
+    from llm_map_reduce_summarizer_amd.engine.engine import LLMEngine
+    from llm_map_reduce_summarizer_amd.engine.registry import load_config
+    path = M.checkpoint("mixed", str(tmp_path / "m"))
+    cfg = load_config(path)
+    assert isinstance(cfg, HybridConfig) and cfg.n_layers == 7 and cfg.layers[2].latent.kv_from == 0
+    assert cfg.n_params() == sum(t.numel() for t in M.weights("mixed").values()) or cfg.n_params() > 0
+    with pytest.raises(ValueError, match="TP"):
+        LLMEngine(cfg, device="cpu", tp_size=2, weights_path=path)
+    c = json.load(open(path + "/config.json"))
+
+    def edited(i, **kw):
+        ls = [dict(la) for la in c["layers"]]
+        ls[i] = dict(ls[i], mixer=dict(ls[i]["mixer"], **kw))
+        return dict(c, layers=ls)
+    for bad in (edited(2, kv_from=1), edited(2, kv_from=2), edited(5, kv_from=2), edited(2, kv_rank=40),
+                edited(0, rot_dim=16), edited(1, kv_heads=3), dict(c, layers=[dict(c["layers"][0], type="else")])):
+        with open(path + "/config.json", "w") as f:
+            json.dump(bad, f)
+        with pytest.raises(ValueError):
+            load_config(path)
+    with open(path + "/config.json", "w") as f:
+        json.dump(edited(0, vdim=48), f)
+    with pytest.raises(ValueError, match="implies"):
+        LLMEngine(load_config(path), device="cpu", weights_path=path)
+    assert get_model_config("tiny-muzozen").state_bytes_per_seq() > 0
+
+
+def test_parameter_count():
+    from llm_map_reduce_summarizer_amd.engine.config import get_model_config
+    from llm_map_reduce_summarizer_amd.engine.hybrid import HybridModel
+    cfg, n = get_model_config("tiny-muzozen"), []
+    m = HybridModel(cfg, torch.device("cpu"), F32)
+
+    def get(name, shape):
+        n.append(math.prod(shape))
+        return torch.zeros(shape)
+    m._fill(get)
+    assert sum(n) == cfg.n_params()
+
+
+def test_trace_runner(tmp_path, monkeypatch, capsys):
+    """bin/trace_run's replay picks the design by config.json."""
+    from llm_map_reduce_summarizer_amd import trace
+    path = M.checkpoint("mixed", str(tmp_path / "m"))
+    ids = M.tokens("mixed", 66)
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": ids[:2], "want": [1]}], "end": []},
+             {"step": 1, "entries": [{"id": "x", "tokens": ids[2:65], "want": []},
+                                     {"id": "y", "tokens": ids[:1], "want": [0]}], "end": ["y"]},
+             {"step": 2, "entries": [{"id": "x", "tokens": ids[65:], "want": [0]}], "end": ["x"]}]
+    monkeypatch.setattr("sys.stdin", io.StringIO("".join(json.dumps(s) + "\n" for s in steps)))
+    assert trace.main(["--model", path, "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "192",
+                       "--device", "cpu"]) == 0
+    assert [ln for ln in capsys.readouterr().out.splitlines() if ln.startswith("done")] == ["done 0", "done 1", "done 2"]
+    got = torch.cat([torch.frombuffer(bytearray((tmp_path / ("%d.f32" % k)).read_bytes()), dtype=F32).view(1, -1)
+                     for k in (0, 1, 2)])
+    M.check(got, M.expected("mixed", ids)[[1, 0, 65]], F32)
+
+
+def test_work_lists_cover_every_row():
+    from llm_map_reduce_summarizer_amd.ops.hip import block_items, delta_chunks, delta_waves
+    for lens, first in (([1, 1, 64, 3], 2), ([1126], 0), ([1000, 70, 600], 0), ([1, 257, 255, 2], 1)):
+        segs, chunks = delta_chunks(lens, first)
+        row = sum(lens[:first])
+        for (i, b, e, c), n, nxt in zip(segs, lens[first:], [s[3] for s in segs[1:]] + [len(chunks)]):
+            assert b == row and e == b + n and lens[i] == n
+            assert [x for ch in chunks[c:nxt] for x in range(*ch)] == list(range(b, e))
+            assert all(hi - lo == 64 for lo, hi in chunks[c:nxt - 1])
+            row = e
+        items = block_items(lens, 256).tolist()
+        assert sorted(map(tuple, items)) == sorted((i, q) for i, n in enumerate(lens) for q in range(0, n, 256))
+        assert [q for _, q in items] == sorted((q for _, q in items), reverse=True)
+    for P, N, pairs in ((128, 128, 256), (128, 128, 32), (64, 128, 512), (16, 32, 4), (136, 200, 999)):
+        assert delta_waves(P, N, pairs) in ((2, 4, 8) if N <= 128 else (2, 4))
+
+
+def test_portion_context_places_every_page():
+    from llm_map_reduce_summarizer_amd import ops
+    ctx = ops.PortionContext([10, 2, 64], [0, 127, 64], [3, 0, 1], torch.device("cpu"))
+    assert ctx.rows == 10 + 129 + 128 and ctx.base.tolist() == [0, 10, 139, 267]
+    assert ctx.pages.tolist() == [[3, 0, 0, 10], [0, 0, 10, 64], [0, 1, 74, 64], [0, 2, 138, 1], [1, 0, 139, 64],
+                                  [1, 1, 203, 64]]
+
+
+def test_command_line_and_throughput_run_muzozen(tmp_path):
+    from llm_map_reduce_summarizer_amd.utils.synth import synthetic_transcript
+    src = tmp_path / "t.json"
+    src.write_text(json.dumps(synthetic_transcript(0.05, seed=3)))
+    out = tmp_path / "s.txt"
+    env = dict(os.environ, CUDA_VISIBLE_DEVICES="", MAX_TOKENS="4", PYTHONPATH=ROOT, OMP_NUM_THREADS="4")
+    path = M.checkpoint("wide", str(tmp_path / "m"))
+    p = subprocess.run([sys.executable, "-m", "llm_map_reduce_summarizer_amd", "-i", str(src), "--provider", "local",
+                        "--model", "tiny-muzozen", "--max-model-len", "2048", "--max-concurrent-requests", "4",
+                        "--max-tokens-per-chunk", "300", "-q", "-o", str(out), "--report"], env=env, cwd="/tmp",
+                       capture_output=True, text=True, timeout=300)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert json.loads(out.with_suffix(".report.json").read_text())["summary"]
+    from llm_map_reduce_summarizer_amd.engine.provider import LocalEngineProvider
+    prov = LocalEngineProvider(path, device="cpu", max_model_len=256, max_num_seqs=2)
+    assert prov.model_config().vocab_size == 130
