@@ -109,7 +109,7 @@ def main() -> int:
                          "(labelled variant, never the headline)")
     ap.add_argument("--throughput", default=None, metavar="MODELS",
                     help="instead of the headline workload: prefill and decode throughput of these models (comma-"
-                         "separated presets, e.g. merulorn-8b,llama3-8b) at a few batch shapes, one JSON line")
+                         "separated presets, e.g. muzozen-8b,merulorn-8b) at a few batch shapes, one JSON line")
     ap.add_argument("--profile", default=None, metavar="DIR", help="torch.profiler trace of the timed steps")
     ap.add_argument("--log-level", default="WARNING")
     args = ap.parse_args()

@@ -39,7 +39,7 @@ def build_parser() -> argparse.ArgumentParser:
     p.add_argument("--output", "-o", help="write the summary here (parent directories are created)")
     p.add_argument("--provider", choices=["local", "mock", "openai", "anthropic"], default=None,
                    help="generation back-end (default: $DEFAULT_PROVIDER, i.e. local)")
-    p.add_argument("--model", help="model name (local: llama3-8b | llama3-70b | merulorn-8b | tiny | a checkpoint folder)")
+    p.add_argument("--model", help="model name (local: llama3-8b | llama3-70b | merulorn-8b | muzozen-8b | tiny | a checkpoint folder)")
     p.add_argument("--max-tokens-per-chunk", type=int, default=4000)
     p.add_argument("--max-concurrent-requests", type=int, default=None)
     p.add_argument("--max-segment-duration", type=int, default=120)
@@ -86,8 +86,9 @@ def build_parser() -> argparse.ArgumentParser:
                         "longer prompts are truncated with a warning")
     e.add_argument("--tokenizer", default=None, help="tiktoken-format vocabulary file (default: bundled)")
     e.add_argument("--weights", default=os.environ.get("MRSUM_WEIGHTS"),
-                   help="safetensors checkpoint for the map model (Hugging Face Llama layout, file or dir, or a Merulorn "
-                        "folder); default: seeded random init.  With a non-preset --model the dir's config.json is used")
+                   help="safetensors checkpoint for the map model (Hugging Face Llama layout, file or dir, or a Merulorn or "
+                        "Muzozen folder); default: seeded random init.  With a non-preset --model the dir's config.json "
+                        "is used")
     e.add_argument("--aggregator-weights", default=None, help="safetensors checkpoint of the aggregator model")
     e.add_argument("--reduce-tp", dest="reduce_tp", action="store_const", const=True, default=None,
                    help="reduce stages tensor-parallel over all ranks (map stays data-parallel); default: on with "

@@ -217,7 +217,7 @@ MRSUM_API int mrsum_embed_bigram(const int* ids, const void* table, const void* 
 
 template <typename T>
 __global__ __launch_bounds__(256) void gelu_cols_kernel(ProjSrc src, int at, int n, T* __restrict__ out, int ldo) {
-    const int t = blockIdx.y, c = 8 * (blockIdx.x * 256 + threadIdx.x);
+    const int t = blockIdx.x, c = 8 * (blockIdx.y * 256 + threadIdx.x);
     if (c >= n) return;
     float v[8];
     proj8<true>(src, t, at + c, v);
@@ -230,9 +230,9 @@ __global__ __launch_bounds__(256) void gelu_cols_kernel(ProjSrc src, int at, int
 MRSUM_API int mrsum_gelu_cols(const float* src, int S, int ld, int T, int at, int n, void* out, int out32, int ldo,
                               hipStream_t s) {
     if (T <= 0 || n <= 0) return 0;
-    if (S < 1 || at % 8 || n % 8 || ld % 8 || ldo % 8 || at + n > ld || T > 65535) return (int)hipErrorInvalidValue;
+    if (S < 1 || at % 8 || n % 8 || ld % 8 || ldo % 8 || at + n > ld) return (int)hipErrorInvalidValue;
     const ProjSrc p{src, S, (size_t)T * ld, ld};
-    const dim3 g(ceil_div(n / 8, 256), T);
+    const dim3 g(T, ceil_div(n / 8, 256));
     if (out32) gelu_cols_kernel<float><<<g, 256, 0, s>>>(p, at, n, (float*)out, ldo);
     else gelu_cols_kernel<bf16><<<g, 256, 0, s>>>(p, at, n, (bf16*)out, ldo);
     return (int)hipGetLastError();

@@ -54,14 +54,17 @@ __device__ __forceinline__ int frag_of(int ib, int jp) { return ib < 2 ? ib : 2 
 // x: convolved rows.  chunks: (first row, end row) of every chunk.  Per (chunk, head): frags [FRAGS] 16-byte pieces,
 // vec [3][64] = 2^c rk | 2^c rq | 2^(c_last - c) rk and 2^(c_last) at [3][0] (stride 256 floats).
 template <int NB>
-__global__ __launch_bounds__(256) void delta_prep_kernel(const bf16* __restrict__ x, DeltaArgs a,
+__global__ __launch_bounds__(256, NB <= 4 ? 4 : 2) void delta_prep_kernel(const bf16* __restrict__ x, DeltaArgs a,
                                                          const int2* __restrict__ chunks, uint4* __restrict__ frags,
                                                          float* __restrict__ vec) {
     constexpr int NN = 32 * NB, LK = NN + 16, LA = Q + 4;
-    __shared__ __attribute__((aligned(16))) bf16 sK[Q * LK];
-    __shared__ __attribute__((aligned(16))) bf16 sQ[Q * LK];
-    __shared__ __attribute__((aligned(16))) float sA[Q * LA];
-    __shared__ __attribute__((aligned(16))) float sT[Q * LA];
+    // the rows' place is taken over by A and T once their dot products are in registers
+    constexpr int ROWS_B = 2 * 2 * Q * LK, AT_B = 2 * 4 * Q * LA;
+    __shared__ __attribute__((aligned(16))) char pool[ROWS_B > AT_B ? ROWS_B : AT_B];
+    bf16* sK = reinterpret_cast<bf16*>(pool);
+    bf16* sQ = sK + Q * LK;
+    float* sA = reinterpret_cast<float*>(pool);
+    float* sT = sA + Q * LA;
     __shared__ __attribute__((aligned(16))) float s_c[Q], s_beta[Q], s_rk[Q], s_rq[Q];
     const int kh = blockIdx.x, ck = blockIdx.y;
     const int2 ch = chunks[ck];
@@ -178,14 +181,16 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const bf16* __restrict_
             }
         __syncthreads();
         {  // diagonal block w: column r16 of its inverse by substitution (lane groups do the same work)
-            const float* ab = sA + 16 * w * LA + 16 * w;
+            int ab = 16 * w * LA + 16 * w;
             float xv[16];
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 float s = r == r16 ? 1.f : 0.f;
 #pragma unroll
-                for (int l = 0; l < r; ++l) s -= ab[r * LA + l] * xv[l];
+                for (int l = 0; l < r; ++l) s -= sA[ab + r * LA + l] * xv[l];
                 xv[r] = s;
+                // rows are read two at a time: all of them read ahead would fill the register file
+                if (r & 1) asm volatile("" : "+v"(ab), "+v"(xv[r]));
             }
 #pragma unroll
             for (int r = 0; r < 16; ++r)

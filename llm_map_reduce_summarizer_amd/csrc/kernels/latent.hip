@@ -29,13 +29,15 @@ struct PrepArgs {
 };
 }  // namespace
 
-// One block per token; a thread holds CH pieces of 8 columns (sections start at multiples of 8; their padding columns
-// are zero in the projection).
-template <bool PARTS, typename T, int CH>
-__global__ __launch_bounds__(1024) void latent_prep_kernel(ProjSrc src, PrepArgs a, T* __restrict__ cq,
-                                                           T* __restrict__ cache) {
+// One block per token, or (WAVE: many rows) one wave; a thread holds CH pieces of 8 columns (sections start at multiples of
+// 8; their padding columns are zero in the projection).
+template <bool PARTS, typename T, int CH, bool WAVE>
+__global__ __launch_bounds__(WAVE ? 256 : 1024) void latent_prep_kernel(ProjSrc src, PrepArgs a, int rows, T* __restrict__ cq,
+                                                                        T* __restrict__ cache) {
     __shared__ float red[64];
-    const int t = blockIdx.x, tid = threadIdx.x, nt = blockDim.x;
+    const int t = WAVE ? 4 * blockIdx.x + (threadIdx.x >> 6) : blockIdx.x;
+    const int tid = WAVE ? threadIdx.x & 63 : threadIdx.x, nt = WAVE ? 64 : blockDim.x;
+    if (WAVE && t >= rows) return;
     const int pq = (a.nq + 7) / 8, pk = a.dkv >= 0 ? (a.nkv + 7) / 8 : 0;
     float v[CH][8];
     float sq = 0.f, sk = 0.f;
@@ -53,11 +55,13 @@ __global__ __launch_bounds__(1024) void latent_prep_kernel(ProjSrc src, PrepArgs
     }
     sq = wave_sum(sq);
     sk = wave_sum(sk);
-    const int lane = tid & 63, nw = nt >> 6;
-    if (lane == 0) { red[tid >> 6] = sq; red[32 + (tid >> 6)] = sk; }
-    __syncthreads();
-    sq = wave_sum(lane < nw ? red[lane] : 0.f);
-    sk = wave_sum(lane < nw ? red[32 + lane] : 0.f);
+    if constexpr (!WAVE) {
+        const int lane = tid & 63, nw = nt >> 6;
+        if (lane == 0) { red[tid >> 6] = sq; red[32 + (tid >> 6)] = sk; }
+        __syncthreads();
+        sq = wave_sum(lane < nw ? red[lane] : 0.f);
+        sk = wave_sum(lane < nw ? red[32 + lane] : 0.f);
+    }
     const float qs = 1.f / sqrtf(sq / (float)a.nq + a.eps);
     T* qo = cq + (size_t)t * a.ldq;
     const int pos = a.positions[t];
@@ -76,8 +80,15 @@ __global__ __launch_bounds__(1024) void latent_prep_kernel(ProjSrc src, PrepArgs
             const int c = 8 * (isq ? p : p - pq), n = isq ? a.nq : a.nkv;
             const float* w = isq ? a.qw : a.kvw;
             const float mul = isq ? qs : ks;
+            if (c + 8 <= n) {
+                float g[8];
+                load8(w + c, g);
 #pragma unroll
-            for (int j = 0; j < 8; ++j) v[i][j] *= c + j < n ? mul * w[c + j] : 0.f;
+                for (int j = 0; j < 8; ++j) v[i][j] *= mul * g[j];
+            } else {
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v[i][j] *= c + j < n ? mul * w[c + j] : 0.f;
+            }
             store8(isq ? qo + c : co + c, v[i]);
         }
     }
@@ -98,12 +109,18 @@ static int launch_prep(const ProjSrc& p, const PrepArgs& a, void* cq, void* cach
     const int pieces = (a.nq + 7) / 8 + (a.dkv >= 0 ? (a.nkv + 7) / 8 : 0);
     const int nt = std::min(1024, ceil_div(pieces, 64) * 64);
     const int ch = ceil_div(pieces, nt);
-#define LP(C) latent_prep_kernel<PARTS, T, C><<<rows, nt, 0, s>>>(p, a, (T*)cq, (T*)cache)
-    if (ch <= 1) LP(1);
+#define LP(C) latent_prep_kernel<PARTS, T, C, false><<<rows, nt, 0, s>>>(p, a, rows, (T*)cq, (T*)cache)
+#define LPW(C) latent_prep_kernel<PARTS, T, C, true><<<ceil_div(rows, 4), 256, 0, s>>>(p, a, rows, (T*)cq, (T*)cache)
+    if (!PARTS && rows >= 1024 && pieces <= 256) {
+        if (pieces <= 64) LPW(1);
+        else if (pieces <= 128) LPW(2);
+        else LPW(4);
+    } else if (ch <= 1) LP(1);
     else if (ch <= 2) LP(2);
     else if (ch <= 4) LP(4);
     else return (int)hipErrorInvalidValue;
 #undef LP
+#undef LPW
     return (int)hipGetLastError();
 }
 
@@ -128,6 +145,7 @@ MRSUM_API int mrsum_latent_prep(const void* src, int S, int ld, int T, int f32, 
 // ------------------------------------------------------------------------------------------------ per-head products
 namespace {
 constexpr int HP_ROWS = 16, HP_COLS = 128;
+constexpr int HM_ROWS = 4, HM_THREADS = 1024, HM_DEPTH = 4;  // merging form: depth up to 128 HM_DEPTH
 
 struct HeadArgs {
     ProjSrc x;        // head h of row t: columns [h * xs, h * xs + xk); SPLITS: unused
@@ -145,16 +163,19 @@ struct HeadArgs {
     const float* po;
     const float* ml;
     int splits;
+    int mrows;        // rows of a merging block, at most HM_ROWS
 };
 }  // namespace
 
-// MODE 0: 16-bit rows, 1: fp32 slabs, 2: split-K partials.  Grid (column blocks + (rot ? 1 : 0), H, 16-row blocks).
+// MODE 0: 16-bit rows, 1: fp32 slabs, 2: split-K partials (fewer rows and more threads a block: merging is a matter of
+// loads in flight).  Grid (column blocks + (rot ? 1 : 0), H, row blocks).
 template <typename T, int MODE>
-__global__ __launch_bounds__(256) void head_product_kernel(const HeadArgs a) {
+__global__ __launch_bounds__(MODE == 2 ? HM_THREADS : 256) void head_product_kernel(const HeadArgs a) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
     T* sx = reinterpret_cast<T*>(smem);
-    const int tid = threadIdx.x, h = blockIdx.y, r0 = blockIdx.z * HP_ROWS;
-    const int nr = min(HP_ROWS, a.rows - r0);
+    const int ROWS = MODE == 2 ? a.mrows : HP_ROWS;
+    const int tid = threadIdx.x, h = blockIdx.y, r0 = blockIdx.z * ROWS;
+    const int nr = min(ROWS, a.rows - r0);
     const int nb = (a.N + HP_COLS - 1) / HP_COLS;
     if ((int)blockIdx.x == nb) {
         if constexpr (MODE != 2) {
@@ -179,11 +200,24 @@ __global__ __launch_bounds__(256) void head_product_kernel(const HeadArgs a) {
     }
     const int ldx = a.K + 8;
     if constexpr (MODE == 2) {
-        __shared__ float sw[HP_ROWS][256];  // weights of the splits, the common denominator divided out
-        const int wv = tid >> 6, lane = tid & 63;
-        for (int r = wv; r < nr; r += 4) {
-            const float2* m = reinterpret_cast<const float2*>(a.ml) + ((size_t)(r0 + r) * a.H + h) * a.splits;
+        __shared__ float sw[HM_ROWS][256];  // weights of the splits, the common denominator divided out
+        __shared__ int s_n[HM_ROWS];        // splits in use: the leading ones
+        __shared__ __attribute__((aligned(16))) float4 part[HM_THREADS];
+        const int wv = tid >> 6, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
+        // this wave's weights, a quarter of the depth of 32 columns, are on their way while the sums are merged
+        const bf16* w = reinterpret_cast<const bf16*>(a.w) + (size_t)h * a.N * a.K + 8 * g;
+        const int n0 = blockIdx.x * HP_COLS + 32 * (wv & 3), kq = 32 * (wv >> 2);
+        u32x4 wf[HM_DEPTH][2];
+#pragma unroll
+        for (int j = 0; j < HM_DEPTH; ++j)
+#pragma unroll
+            for (int q = 0; q < 2; ++q)
+                wf[j][q] = *reinterpret_cast<const u32x4*>(w + (size_t)min(n0 + 16 * q + r16, a.N - 1) * a.K +
+                                                           min(kq + 128 * j, a.K - 32));
+        if (wv < nr) {
+            const float2* m = reinterpret_cast<const float2*>(a.ml) + ((size_t)(r0 + wv) * a.H + h) * a.splits;
             float mx[4], sm[4], best = -INFINITY;
+            int n = 0;
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 const int sp = lane + 64 * q;
@@ -191,6 +225,7 @@ __global__ __launch_bounds__(256) void head_product_kernel(const HeadArgs a) {
                 mx[q] = v.x;
                 sm[q] = v.y;
                 best = fmaxf(best, v.x);
+                n += __popcll(__ballot(v.x != -INFINITY));
             }
             best = wave_max(best);
             float den = 0.f;
@@ -201,24 +236,63 @@ __global__ __launch_bounds__(256) void head_product_kernel(const HeadArgs a) {
             }
             den = wave_sum(den);
 #pragma unroll
-            for (int q = 0; q < 4; ++q) sw[r][lane + 64 * q] = mx[q] / den;
+            for (int q = 0; q < 4; ++q) sw[wv][lane + 64 * q] = mx[q] / den;
+            if (lane == 0) s_n[wv] = n;
         }
         __syncthreads();
-        const int v4 = a.K / 4;
-        for (int i = tid; i < HP_ROWS * v4; i += 256) {
-            const int r = i / v4, k = 4 * (i % v4);
+        // thread = (share of the splits, row, four columns)
+        const int v4 = a.xk / 4, items = nr * v4, shares = HM_THREADS / items;
+        const int sh = tid / items, r = tid % items / v4, k = 4 * (tid % v4);
+        if (sh < shares) {
             float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (r < nr && k < a.xk) {
-                const float* p = a.po + ((size_t)(r0 + r) * a.H + h) * a.splits * a.xk + k;
+            const float* p = a.po + ((size_t)(r0 + r) * a.H + h) * a.splits * a.xk + k;
+            const int ns = s_n[r];
 #pragma unroll 8
-                for (int sp = 0; sp < a.splits; ++sp) {
-                    const float4 v = *reinterpret_cast<const float4*>(p + (size_t)sp * a.xk);
-                    const float w = sw[r][sp];
-                    acc.x += w * v.x; acc.y += w * v.y; acc.z += w * v.z; acc.w += w * v.w;
-                }
+            for (int sp = sh; sp < ns; sp += shares) {
+                const float4 v = *reinterpret_cast<const float4*>(p + (size_t)sp * a.xk);
+                const float f = sw[r][sp];
+                acc.x += f * v.x; acc.y += f * v.y; acc.z += f * v.z; acc.w += f * v.w;
             }
-            store4(sx + r * ldx + k, acc);
+            part[tid] = acc;
         }
+        __syncthreads();
+        for (int i = tid; i < HP_ROWS * (a.K / 4); i += HM_THREADS) {
+            const int row = i / (a.K / 4), c = i % (a.K / 4);
+            float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (row < nr && c < v4)
+                for (int q = 0; q < shares; ++q) {
+                    const float4 v = part[q * items + row * v4 + c];
+                    acc.x += v.x; acc.y += v.y; acc.z += v.z; acc.w += v.w;
+                }
+            store4(sx + row * ldx + 4 * c, acc);
+        }
+        __syncthreads();
+        f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int j = 0; j < HM_DEPTH; ++j)
+            if (kq + 128 * j < a.K) {
+                const bf16x8 xf = *reinterpret_cast<const bf16x8*>(sx + r16 * ldx + 8 * g + kq + 128 * j);
+#pragma unroll
+                for (int q = 0; q < 2; ++q)
+                    acc[q] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wf[j][q]), xf, acc[q], 0, 0, 0);
+            }
+        // the four quarters of the depth: rows of four lanes each
+        f32x4* quarter = reinterpret_cast<f32x4*>(part);
+        if (r16 < HM_ROWS)
+#pragma unroll
+            for (int q = 0; q < 2; ++q) quarter[(wv * 2 + q) * 16 + 4 * g + r16] = acc[q];
+        __syncthreads();
+        if (tid < 128 * HM_ROWS / 4) {  // thread = (16-column group, lane group, row)
+            const int c16 = tid >> 4, gg = (tid >> 2) & 3, row = tid & 3;
+            const int n = blockIdx.x * HP_COLS + 16 * c16 + 4 * gg;  // N % 8 == 0
+            f32x4 y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < 4; ++kk) y += quarter[((4 * kk + (c16 >> 1)) * 2 + (c16 & 1)) * 16 + 4 * gg + row];
+            if (row < nr && n < a.N)
+                store4(reinterpret_cast<T*>(a.out) + (size_t)(r0 + row) * a.ldo + h * a.os + n,
+                       make_float4(y[0], y[1], y[2], y[3]));
+        }
+        return;
     } else {
         const int v8 = a.K / 8;
         for (int i = tid; i < HP_ROWS * v8; i += 256) {
@@ -281,16 +355,20 @@ MRSUM_API int mrsum_head_product(const void* x, int S, int ldx, int xrows, int r
                                  hipStream_t s) {
     if (rows <= 0) return 0;
     if (N <= 0 || N % 8 || K % 32 || xk % 8 || xk > K || os % 4 || ldo % 4 || H <= 0 || H > 65535 || rot % 2 ||
-        ceil_div(rows, HP_ROWS) > 65535 || (S < 0 && (f32 || rot || !po || !ml || splits < 1 || splits > 256)) ||
+        ceil_div(rows, S < 0 ? 1 : HP_ROWS) > 65535 ||
+        (S < 0 && (f32 || rot || !po || !ml || splits < 1 || splits > 256 || HM_ROWS * (xk / 4) > HM_THREADS || K > 128 * HM_DEPTH)) ||
         (S >= 0 && (rows > xrows || ldx % 8 || xs % 8)) || (f32 && S < 1))
         return (int)hipErrorInvalidValue;
+    // as few rows a block as fill the CUs
+    const int mrows = std::max(1, std::min(HM_ROWS, rows * H / 256));
     const HeadArgs a{ProjSrc{x, S, (size_t)xrows * ldx, ldx}, xs, xk, w, N, K, out, os, ldo, rows, H, rot, rot8, rx, ro,
-                     (const float2*)cs, positions, po, ml, splits};
-    const dim3 g(ceil_div(N, HP_COLS) + (rot ? 1 : 0), H, ceil_div(rows, HP_ROWS));
+                     (const float2*)cs, positions, po, ml, splits, mrows};
+    const int rb = S < 0 ? mrows : HP_ROWS;
+    const dim3 g(ceil_div(N, HP_COLS) + (rot ? 1 : 0), H, ceil_div(rows, rb));
     const size_t lds = (size_t)HP_ROWS * (K + 8) * (f32 ? 4 : 2);
     if (lds > 40 * 1024) return (int)hipErrorInvalidValue;
     if (f32) head_product_kernel<float, 1><<<g, 256, lds, s>>>(a);
-    else if (S < 0) head_product_kernel<bf16, 2><<<g, 256, lds, s>>>(a);
+    else if (S < 0) head_product_kernel<bf16, 2><<<g, HM_THREADS, lds, s>>>(a);
     else if (S) head_product_kernel<bf16, 1><<<g, 256, lds, s>>>(a);
     else head_product_kernel<bf16, 0><<<g, 256, lds, s>>>(a);
     return (int)hipGetLastError();

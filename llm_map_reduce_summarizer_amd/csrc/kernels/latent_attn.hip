@@ -8,8 +8,9 @@
 //
 // latent_decode: split-K attention of single tokens with absorbed queries over the cached rows themselves (one row per
 // token for all heads; its first columns are also the value).  A workgroup runs up to 32 heads of one sequence over its
-// share of pages: a page's rows sit in LDS (the next page's in registers), every wave scores a 16-key x 16-head tile, and
-// after the scores have crossed LDS every wave weights its own block of value columns.  Output: unmerged partial sums.
+// share of pages: a page's rows sit in LDS (the next page's in registers), every wave scores and exponentiates a 16-key x
+// 16-head tile, and after the weights have crossed LDS every wave sums its own block of value columns.  Output: unmerged
+// partial sums.
 #include "common.h"
 
 namespace {
@@ -258,31 +259,23 @@ struct LatDecode {
 };
 }  // namespace
 
-// KB: 32-column blocks of a cached row, VB: 128-column blocks of the latent.  Grid (S, ceil(H / 32), B).
+// KB: 32-column blocks of a cached row, VB: 128-column blocks of the latent.  Grid (S, ceil(H / 32), B).  Two barriers a
+// page: the next page's registers go to the other LDS stage between them, when every wave is past the page before.
 template <int KB, int VB>
 __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a) {
-    constexpr int LK = 32 * KB + 8, LS = BN + 4, IT = KB / 2;
-    __shared__ __attribute__((aligned(16))) bf16 sk[BN * LK];
-    __shared__ __attribute__((aligned(16))) float ss[DH * LS];
+    constexpr int LK = 32 * KB + 8, LP = BN + 8, IT = KB / 2;
+    __shared__ __attribute__((aligned(16))) bf16 sk[2][BN * LK];
+    __shared__ __attribute__((aligned(16))) bf16 sph[DH * LP];  // softmax weights, hi and lo terms
+    __shared__ __attribute__((aligned(16))) bf16 spl[DH * LP];
+    __shared__ __attribute__((aligned(16))) float smax[DH][4];  // maxima of the four 16-key blocks
     const int sp = blockIdx.x, h0 = DH * blockIdx.y, b = blockIdx.z;
     const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4, q4 = r16 >> 2, p4 = 4 * (r16 & 3);
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6), kb4 = w & 3, hb = w >> 2;
-    const int pos = a.positions[b], pages = pos / BN + 1, per = (pages + a.S - 1) / a.S;
-    const int p0 = min(sp * per, pages), p1 = min(p0 + per, pages);
+    const int pos = a.positions[b], pages = pos / BN + 1;
+    const int used = min(a.S, pages);  // splits past them are empty
+    const int p0 = sp < used ? (int)((long long)pages * sp / used) : 0;
+    const int p1 = sp < used ? (int)((long long)pages * (sp + 1) / used) : 0;
     const int* bt = a.bt + (size_t)b * a.bt_stride;
-    bf16x8 qf[KB];  // this wave's 16 heads
-    {
-        const int h = h0 + 16 * hb + r16;
-        const bf16* qp = a.q + ((size_t)b * a.H + min(h, a.H - 1)) * a.row;
-#pragma unroll
-        for (int kb = 0; kb < KB; ++kb) {
-            const int c = 32 * kb + 8 * g;
-            u32x4 v = *reinterpret_cast<const u32x4*>(qp + min(c, a.row - 8));
-            if (c >= a.row || h >= a.H) v = u32x4{0, 0, 0, 0};
-            qf[kb] = as8(v);
-        }
-    }
-    for (int i = tid; i < BN * LK / 8; i += 512) *reinterpret_cast<u32x4*>(sk + 8 * i) = u32x4{0, 0, 0, 0};
     const int rc = a.row / 8, total = BN * rc;  // 16-byte pieces of a row / of a page
     u32x4 reg[IT];
     int at[IT];  // LDS offset of piece tid + 512 i (past the page: the last piece once more)
@@ -298,69 +291,111 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
             reg[i] = *reinterpret_cast<const u32x4*>(pg_ + 8 * min(tid + 512 * i, total - 1));          \
     }
     f32x4 acc[VB][2];
-    float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
+    float m[2] = {-INFINITY, -INFINITY}, l = 0.f;  // maxima of heads r16, 16 + r16; this lane's share of head 16 hb + r16's sum
 #pragma unroll
     for (int vb = 0; vb < VB; ++vb) acc[vb][0] = acc[vb][1] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (p0 < p1) LOAD_PAGE(p0)
-    for (int p = p0; p < p1; ++p) {
-        __syncthreads();  // every wave is done with the previous page (first round: the zeros are in)
-#pragma unroll
-        for (int i = 0; i < IT; ++i) *reinterpret_cast<u32x4*>(sk + at[i]) = reg[i];
-        __syncthreads();
-        LOAD_PAGE(min(p + 1, p1 - 1))
+    if (p0 < p1) {
+        LOAD_PAGE(p0)
+        bf16x8 qf[KB];  // this wave's 16 heads
         {
-            f32x4 s[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
-            const bf16* kr = sk + (16 * kb4 + r16) * LK + 8 * g;
+            const int h = h0 + 16 * hb + r16;
+            const bf16* qp = a.q + ((size_t)b * a.H + min(h, a.H - 1)) * a.row;
 #pragma unroll
-            for (int kb = 0; kb < KB; ++kb)
-                s[kb & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kr + 32 * kb), qf[kb],
-                                                                    s[kb & 1], 0, 0, 0);
-            *reinterpret_cast<f32x4*>(ss + (16 * hb + r16) * LS + 16 * kb4 + 4 * g) = s[0] + s[1];
+            for (int kb = 0; kb < KB; ++kb) {
+                const int c = 32 * kb + 8 * g;
+                u32x4 v = *reinterpret_cast<const u32x4*>(qp + min(c, a.row - 8));
+                if (c >= a.row || h >= a.H) v = u32x4{0, 0, 0, 0};
+                qf[kb] = as8(v);
+            }
         }
+        // columns past the row: zeros in both stages
+        const int rz = 4 * KB + 1 - rc;
+        for (int i = tid; i < 2 * BN * rz; i += 512)
+            *reinterpret_cast<u32x4*>(&sk[0][0] + (i / rz) * LK + 8 * (rc + i % rz)) = u32x4{0, 0, 0, 0};
+#pragma unroll
+        for (int i = 0; i < IT; ++i) *reinterpret_cast<u32x4*>(&sk[0][0] + at[i]) = reg[i];
+        LOAD_PAGE(min(p0 + 1, p1 - 1))
         __syncthreads();
-        const int kmax = pos - BN * p;  // last visible key of the page
-        bf16x8 ph[2][2], pl[2][2];
+        for (int p = p0; p < p1; ++p) {
+            const bf16* cur = &sk[(p - p0) & 1][0];
+            f32x4 s;
+            {
+                f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+                const bf16* kr = cur + (16 * kb4 + r16) * LK + 8 * g;
 #pragma unroll
-        for (int hh = 0; hh < 2; ++hh) {
-            float v[2][8], mx = -INFINITY;
-#pragma unroll
-            for (int kk = 0; kk < 2; ++kk) {
-                load8(ss + (16 * hh + r16) * LS + 32 * kk + 8 * g, v[kk]);
-#pragma unroll
-                for (int j = 0; j < 8; ++j) {
-                    v[kk][j] = 32 * kk + 8 * g + j <= kmax ? v[kk][j] * a.scale_log2 : -INFINITY;
-                    mx = fmaxf(mx, v[kk][j]);
+                for (int kb = 0; kb < KB; kb += 2) {
+                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kr + 32 * kb), qf[kb], s0,
+                                                                 0, 0, 0);
+                    s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kr + 32 * kb + 32),
+                                                                 qf[kb + 1], s1, 0, 0, 0);
                 }
+                s = s0 + s1;
+            }
+            const int kmax = pos - BN * p - 16 * kb4 - 4 * g;  // last visible of this lane's four keys
+            float mx = -INFINITY;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                s[j] = j <= kmax ? s[j] * a.scale_log2 : -INFINITY;
+                mx = fmaxf(mx, s[j]);
             }
             mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-            const float mn = fmaxf(m[hh], mx), alpha = __builtin_amdgcn_exp2f(m[hh] - mn);  // key 0 of a page is visible
-            m[hh] = mn;
-            l[hh] *= alpha;
+            if (g == 0) smax[16 * hb + r16][kb4] = mx;
+            __syncthreads();
+            float alpha[2];
 #pragma unroll
-            for (int kk = 0; kk < 2; ++kk)
+            for (int hh = 0; hh < 2; ++hh) {
+                const f32x4 v = *reinterpret_cast<const f32x4*>(&smax[16 * hh + r16][0]);
+                const float mn = fmaxf(m[hh], fmaxf(fmaxf(v[0], v[1]), fmaxf(v[2], v[3])));  // key 0 of a page is visible
+                alpha[hh] = __builtin_amdgcn_exp2f(m[hh] - mn);
+                m[hh] = mn;
+            }
+            {
+                const float mh = hb ? m[1] : m[0];
+                float e[4], lo[4];
 #pragma unroll
-                for (int j = 0; j < 8; ++j) {
-                    const float e = __builtin_amdgcn_exp2f(v[kk][j] - mn);
-                    l[hh] += e;
-                    ph[hh][kk][j] = (bf16)e;
-                    pl[hh][kk][j] = (bf16)(e - (float)ph[hh][kk][j]);
-                }
+                for (int j = 0; j < 4; ++j) e[j] = __builtin_amdgcn_exp2f(s[j] - mh);
+                l = l * (hb ? alpha[1] : alpha[0]) + (e[0] + e[1]) + (e[2] + e[3]);
 #pragma unroll
-            for (int vb = 0; vb < VB; ++vb) acc[vb][hh] *= alpha;
-        }
+                for (int j = 0; j < 4; ++j) lo[j] = e[j] - (float)(bf16)e[j];
+                const int o = (16 * hb + r16) * LP + 16 * kb4 + 4 * g;
+                *reinterpret_cast<uint2*>(sph + o) = make_uint2(pack2(e[0], e[1]), pack2(e[2], e[3]));
+                *reinterpret_cast<uint2*>(spl + o) = make_uint2(pack2(lo[0], lo[1]), pack2(lo[2], lo[3]));
+            }
+            if (p + 1 < p1) {
+                bf16* nxt = &sk[(p - p0 + 1) & 1][0];
 #pragma unroll
-        for (int vb = 0; vb < VB; ++vb) {
-            const int r0 = 16 * (w + 8 * vb);
-            if (r0 < a.rank) {
+                for (int i = 0; i < IT; ++i) *reinterpret_cast<u32x4*>(nxt + at[i]) = reg[i];
+                LOAD_PAGE(min(p + 2, p1 - 1))
+            }
+#pragma unroll
+            for (int vb = 0; vb < VB; ++vb) {
+                acc[vb][0] *= alpha[0];
+                acc[vb][1] *= alpha[1];
+            }
+            __syncthreads();
+            bf16x8 ph[2][2], pl[2][2];
+#pragma unroll
+            for (int hh = 0; hh < 2; ++hh)
 #pragma unroll
                 for (int kk = 0; kk < 2; ++kk) {
-                    const bf16* vr = sk + (32 * kk + 8 * g + q4) * LK + r0 + p4;
-                    const bf16x8 vt = tr8(vr, vr + 4 * LK);
+                    const int o = (16 * hh + r16) * LP + 32 * kk + 8 * g;
+                    ph[hh][kk] = *reinterpret_cast<const bf16x8*>(sph + o);
+                    pl[hh][kk] = *reinterpret_cast<const bf16x8*>(spl + o);
+                }
 #pragma unroll
-                    for (int hh = 0; hh < 2; ++hh) {
-                        acc[vb][hh] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, ph[hh][kk], acc[vb][hh], 0, 0, 0);
-                        acc[vb][hh] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pl[hh][kk], acc[vb][hh], 0, 0, 0);
+            for (int vb = 0; vb < VB; ++vb) {
+                const int r0 = 16 * (w + 8 * vb);
+                if (r0 < a.rank) {
+#pragma unroll
+                    for (int kk = 0; kk < 2; ++kk) {
+                        const bf16* vr = cur + (32 * kk + 8 * g + q4) * LK + r0 + p4;
+                        const bf16x8 vt = tr8(vr, vr + 4 * LK);
+#pragma unroll
+                        for (int hh = 0; hh < 2; ++hh) {
+                            acc[vb][hh] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, ph[hh][kk], acc[vb][hh], 0, 0, 0);
+                            acc[vb][hh] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, pl[hh][kk], acc[vb][hh], 0, 0, 0);
+                        }
                     }
                 }
             }
@@ -370,7 +405,7 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
 #pragma unroll
     for (int hh = 0; hh < 2; ++hh) {
         const int h = h0 + 16 * hh + r16;
-        if (h >= a.H) continue;
+        if (h >= a.H || p0 == p1) continue;
         const size_t e = ((size_t)b * a.H + h) * a.S + sp;
 #pragma unroll
         for (int vb = 0; vb < VB; ++vb) {
@@ -378,12 +413,17 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
             if (r < a.rank) *reinterpret_cast<f32x4*>(a.po + e * a.rank + r) = acc[vb][hh];
         }
     }
-#pragma unroll
-    for (int hh = 0; hh < 2; ++hh) {
-        l[hh] += __shfl_xor(l[hh], 16, 64);
-        l[hh] += __shfl_xor(l[hh], 32, 64);
-        const int h = h0 + 16 * hh + r16;
-        if (w == 0 && g == 0 && h < a.H) a.ml[((size_t)b * a.H + h) * a.S + sp] = make_float2(m[hh], l[hh]);
+    // the sum of a head: lane groups, then the four key blocks (waves of the same half)
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    __syncthreads();
+    if (g == 0) smax[16 * hb + r16][kb4] = l;
+    __syncthreads();
+    if (tid < 2 * 64 && g == 0) {
+        const int hh = w, h = h0 + 16 * hh + r16;
+        const f32x4 v = *reinterpret_cast<const f32x4*>(&smax[16 * hh + r16][0]);
+        if (h < a.H)
+            a.ml[((size_t)b * a.H + h) * a.S + sp] = make_float2(hh ? m[1] : m[0], (v[0] + v[1]) + (v[2] + v[3]));
     }
 }
 

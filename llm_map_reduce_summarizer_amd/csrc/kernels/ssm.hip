@@ -346,17 +346,24 @@ __device__ __forceinline__ float4 gated4(const float* y, const float4& z) {
                        v.z * z.z * logistic_for<T>(z.z), v.w * z.w * logistic_for<T>(z.w));
 }
 
-// L lanes per norm group, VPT float4 each in registers (VPT = 0: any part size, re-read for the second pass).  L = 64:
-// a wave per group, four groups per block; L = 256 / 1024: one block per group (few rows: all loads in flight).
+template <int L>
+__device__ __forceinline__ float lanes_sum(float v) {
+#pragma unroll
+    for (int o = L / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+    return v;
+}
+
+// L lanes per norm group, VPT float4 each in registers (VPT = 0: any part size, re-read for the second pass).  L <= 64:
+// a wave or part of one per group; L = 256 / 1024: one block per group (few rows: all loads in flight).
 // POST: the norm first, then the gate, and one weight vector shared by the groups (heads).  Columns from col + n to
 // zero_to are zeroed.
 template <bool PARTS, typename TO, int L, int VPT, bool POST>
-__global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const float* __restrict__ y, ProjSrc u, int z_at,
+__global__ __launch_bounds__(L <= 64 ? 256 : L) void gated_norm_kernel(const float* __restrict__ y, ProjSrc u, int z_at,
                                                                        const float* __restrict__ w, int n, int groups,
                                                                        float eps, float out_scale, TO* __restrict__ out,
                                                                        int ldo, int col, int zero_to) {
     __shared__ float red[16];
-    constexpr int GPB = L == 64 ? 4 : 1;
+    constexpr int GPB = L <= 64 ? 256 / L : 1;
     const int gb = (groups + GPB - 1) / GPB;
     const int t = blockIdx.x / gb, g0 = (blockIdx.x % gb) * GPB;
     const int l = threadIdx.x % L, g = g0 + threadIdx.x / L;
@@ -368,16 +375,18 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
     const bool on = g < groups;
     float ss = 0.f;
     if constexpr (VPT > 0) {
-        float4 v[VPT];
+        float4 v[VPT], z[POST ? VPT : 1];
 #pragma unroll
         for (int i = 0; i < VPT; ++i) {
             const int c = 4 * (l + L * i);
             v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (on && c < ng)
+            if (on && c < ng) {
                 v[i] = POST ? *reinterpret_cast<const float4*>(yr + c) : gated4<TO>(yr + c, proj4<PARTS>(u, t, zc + c));
+                if constexpr (POST) z[i] = proj4<PARTS>(u, t, zc + c);
+            }
             ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
         }
-        ss = L == 64 ? wave_sum(ss) : block_sum(ss, red);
+        ss = L <= 64 ? lanes_sum<(L <= 64 ? L : 64)>(ss) : block_sum(ss, red);
         const float inv = out_scale / sqrtf(ss / (float)ng + eps);
 #pragma unroll
         for (int i = 0; i < VPT; ++i) {
@@ -385,9 +394,8 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
             if (on && c < ng) {
                 float4 k = *reinterpret_cast<const float4*>(wr + c);
                 if constexpr (POST) {
-                    const float4 z = proj4<PARTS>(u, t, zc + c);
-                    k.x *= z.x * logistic_for<TO>(z.x); k.y *= z.y * logistic_for<TO>(z.y);
-                    k.z *= z.z * logistic_for<TO>(z.z); k.w *= z.w * logistic_for<TO>(z.w);
+                    k.x *= z[i].x * logistic_for<TO>(z[i].x); k.y *= z[i].y * logistic_for<TO>(z[i].y);
+                    k.z *= z[i].z * logistic_for<TO>(z[i].z); k.w *= z[i].w * logistic_for<TO>(z[i].w);
                 }
                 store4(o + c, make_float4(v[i].x * inv * k.x, v[i].y * inv * k.y, v[i].z * inv * k.z, v[i].w * inv * k.w));
             }
@@ -397,7 +405,7 @@ __global__ __launch_bounds__(L == 64 ? 256 : L) void gated_norm_kernel(const flo
             const float z = POST ? 0.f : proj_at<PARTS>(u, t, zc + c), v = POST ? yr[c] : yr[c] * z * logistic(z);
             ss += v * v;
         }
-        ss = L == 64 ? wave_sum(ss) : block_sum(ss, red);
+        ss = L <= 64 ? lanes_sum<(L <= 64 ? L : 64)>(ss) : block_sum(ss, red);
         const float inv = out_scale / sqrtf(ss / (float)ng + eps);
         for (int c = l; on && c < ng; c += L) {
             const float z = proj_at<PARTS>(u, t, zc + c);
@@ -412,13 +420,15 @@ template <bool POST>
 static int launch_gated_norm(const float* y, const ProjSrc& p, int T, int z_at, const float* w, int n, int groups, float eps,
                              float out_scale, void* out, int out32, int ldo, int col, int zero_to, hipStream_t s) {
     const int ng = n / groups, q = ng % 4 ? 0 : ng / 4;  // float4 per part (0: unaligned parts)
-    const long long gb = groups, gw = (groups + 3) / 4;
+    const long long gb = groups, gw = (groups + 3) / 4, gn = (groups + 15) / 16, gh = (groups + 7) / 8;
     if ((long long)T * groups > 0x7fffffff) return (int)hipErrorInvalidValue;
 #define GN(PT, TO, L_, V, NB_) \
-    gated_norm_kernel<PT, TO, L_, V, POST><<<(int)((long long)T * (NB_)), L_ == 64 ? 256 : L_, 0, s>>>(                  \
+    gated_norm_kernel<PT, TO, L_, V, POST><<<(int)((long long)T * (NB_)), L_ <= 64 ? 256 : L_, 0, s>>>(                  \
         y, p, z_at, w, n, groups, eps, out_scale, (TO*)out, ldo, col, zero_to)
 #define GN_L(PT, TO)                                        \
     if (!q || q > 4096) GN(PT, TO, 256, 0, gb);             \
+    else if (q <= 16 && T > 512) GN(PT, TO, 16, 1, gn);     \
+    else if (q <= 32 && T > 512) GN(PT, TO, 32, 1, gh);     \
     else if (q <= 64 && T > 512) GN(PT, TO, 64, 1, gw);     \
     else if (q <= 256 && T > 512) GN(PT, TO, 64, 4, gw);    \
     else if (q <= 256) GN(PT, TO, 256, 1, gb);              \

@@ -1761,6 +1761,7 @@ def project_gelu(x, w, n: int, out, col: int, cols: int):
 # (16-column key steps, key width, value width) of the instantiated prompt-portion kernels (latent_attn.hip)
 LATENT_FORMS = ((4, 64, 64), (8, 128, 128), (12, 192, 128))
 LATENT_BLOCK = 256  # query rows per workgroup
+LATENT_SPLIT_PAGES = 2  # pages of a decode split at least: shorter ones cost more to merge than they save
 LATENT_DECODE_FORMS = ((128, 128), (256, 320), (512, 576))  # (latent width, row width)
 
 
@@ -1782,11 +1783,11 @@ def block_items(lens, rows: int) -> torch.Tensor:
 
 class LatentWorkspace:
     """Split-K partial sums of latent_decode for ``B`` rows whose contexts reach ``max_ctx``: as many (sequence, head
-    block, split) workgroups as there are CUs (one fits a CU), at least a page each."""
+    block, split) workgroups as there are CUs (one fits a CU)."""
 
     def __init__(self, B: int, heads: int, rank: int, max_ctx: int, device):
         groups = max(1, B * -(-heads // 32))
-        self.splits = max(1, min(N_CU // groups, -(-max_ctx // 64), 256))
+        self.splits = max(1, min(N_CU // groups, -(-max_ctx // (64 * LATENT_SPLIT_PAGES)), 256))
         self.part_o = torch.empty(B * heads * self.splits * rank, dtype=torch.float32, device=device)
         self.part_ml = torch.empty(B * heads * self.splits * 2, dtype=torch.float32, device=device)
 
