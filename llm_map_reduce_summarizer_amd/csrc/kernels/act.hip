@@ -216,24 +216,19 @@ MRSUM_API int mrsum_embed_bigram(const int* ids, const void* table, const void* 
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void gelu_cols_kernel(ProjSrc src, int at, int n, T* __restrict__ out, int ldo) {
-    const int t = blockIdx.x, c = 8 * (blockIdx.y * 256 + threadIdx.x);
-    if (c >= n) return;
-    float v[8];
-    proj8<true>(src, t, at + c, v);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = gelu_tanh<T>(v[j]);
-    store8(out + (size_t)t * ldo + c, v);
+__global__ __launch_bounds__(256) void gelu_cols_kernel(ProjSrc src, GeluJob job) {
+    gelu_piece<true, T>(src, job, blockIdx.x, 8 * (blockIdx.y * 256 + threadIdx.x));
 }
 
 // columns [at, at + n) of fp32 slabs [S][T][ld] -> out rows of stride ldo (bf16, or fp32 with out32)
 MRSUM_API int mrsum_gelu_cols(const float* src, int S, int ld, int T, int at, int n, void* out, int out32, int ldo,
                               hipStream_t s) {
     if (T <= 0 || n <= 0) return 0;
-    if (S < 1 || at % 8 || n % 8 || ld % 8 || ldo % 8 || at + n > ld) return (int)hipErrorInvalidValue;
+    const GeluJob job{at, n, ldo, out};
+    if (ld % 8 || !gelu_job_ok(job, S, ld)) return (int)hipErrorInvalidValue;
     const ProjSrc p{src, S, (size_t)T * ld, ld};
     const dim3 g(T, ceil_div(n / 8, 256));
-    if (out32) gelu_cols_kernel<float><<<g, 256, 0, s>>>(p, at, n, (float*)out, ldo);
-    else gelu_cols_kernel<bf16><<<g, 256, 0, s>>>(p, at, n, (bf16*)out, ldo);
+    if (out32) gelu_cols_kernel<float><<<g, 256, 0, s>>>(p, job);
+    else gelu_cols_kernel<bf16><<<g, 256, 0, s>>>(p, job);
     return (int)hipGetLastError();
 }

@@ -211,4 +211,26 @@ __device__ __forceinline__ float gelu_tanh(float z) {
     return z * logistic_for<T>(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
 
+
 static inline int ceil_div(int a, int b) { return (a + b - 1) / b; }
+
+// Columns [at, at + n) of a projection's slabs through gelu into rows out + t * ldo (n = 0: nothing): a job that kernels
+// with few rows take along in blocks of their own.
+struct GeluJob {
+    int at, n, ldo;
+    void* out;
+};
+
+template <bool PARTS, typename T>
+__device__ __forceinline__ void gelu_piece(const ProjSrc& src, const GeluJob& j, int t, int c) {
+    if (c >= j.n) return;
+    float v[8];
+    proj8<PARTS>(src, t, j.at + c, v);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v[k] = gelu_tanh<T>(v[k]);
+    store8(reinterpret_cast<T*>(j.out) + (size_t)t * j.ldo + c, v);
+}
+
+static inline bool gelu_job_ok(const GeluJob& j, int S, int ld) {
+    return j.n == 0 || (S >= 1 && j.n > 0 && j.out && j.at >= 0 && j.at % 8 == 0 && j.n % 8 == 0 && j.ldo % 8 == 0 && j.at + j.n <= ld);
+}

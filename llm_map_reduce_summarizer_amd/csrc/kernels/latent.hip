@@ -33,8 +33,14 @@ struct PrepArgs {
 // 8; their padding columns are zero in the projection).
 template <bool PARTS, typename T, int CH, bool WAVE>
 __global__ __launch_bounds__(WAVE ? 256 : 1024) void latent_prep_kernel(ProjSrc src, PrepArgs a, int rows, T* __restrict__ cq,
-                                                                        T* __restrict__ cache) {
+                                                                        T* __restrict__ cache, GeluJob job) {
     __shared__ float red[64];
+    if constexpr (PARTS && !WAVE) {
+        if (blockIdx.y) {
+            gelu_piece<true, T>(src, job, blockIdx.x, 8 * ((blockIdx.y - 1) * blockDim.x + threadIdx.x));
+            return;
+        }
+    }
     const int t = WAVE ? 4 * blockIdx.x + (threadIdx.x >> 6) : blockIdx.x;
     const int tid = WAVE ? threadIdx.x & 63 : threadIdx.x, nt = WAVE ? 64 : blockDim.x;
     if (WAVE && t >= rows) return;
@@ -105,12 +111,14 @@ __global__ __launch_bounds__(WAVE ? 256 : 1024) void latent_prep_kernel(ProjSrc 
 }
 
 template <bool PARTS, typename T>
-static int launch_prep(const ProjSrc& p, const PrepArgs& a, void* cq, void* cache, int rows, hipStream_t s) {
+static int launch_prep(const ProjSrc& p, const PrepArgs& a, void* cq, void* cache, int rows, const GeluJob& job,
+                       hipStream_t s) {
     const int pieces = (a.nq + 7) / 8 + (a.dkv >= 0 ? (a.nkv + 7) / 8 : 0);
     const int nt = std::min(1024, ceil_div(pieces, 64) * 64);
     const int ch = ceil_div(pieces, nt);
-#define LP(C) latent_prep_kernel<PARTS, T, C, false><<<rows, nt, 0, s>>>(p, a, rows, (T*)cq, (T*)cache)
-#define LPW(C) latent_prep_kernel<PARTS, T, C, true><<<ceil_div(rows, 4), 256, 0, s>>>(p, a, rows, (T*)cq, (T*)cache)
+    const dim3 grid(rows, 1 + ceil_div(job.n / 8, nt));
+#define LP(C) latent_prep_kernel<PARTS, T, C, false><<<grid, nt, 0, s>>>(p, a, rows, (T*)cq, (T*)cache, job)
+#define LPW(C) latent_prep_kernel<PARTS, T, C, true><<<ceil_div(rows, 4), 256, 0, s>>>(p, a, rows, (T*)cq, (T*)cache, job)
     if (!PARTS && rows >= 1024 && pieces <= 256) {
         if (pieces <= 64) LPW(1);
         else if (pieces <= 128) LPW(2);
@@ -125,21 +133,24 @@ static int launch_prep(const ProjSrc& p, const PrepArgs& a, void* cq, void* cach
 }
 
 // src: S = 0 bf16 rows [T][ld], S >= 1 fp32 slabs.  f32: cq / cache fp32 (slabs only), else bf16.  dkv < 0: query
-// latents only.
+// latents only.  g_n > 0: columns of the slabs through gelu besides (GeluJob).
 MRSUM_API int mrsum_latent_prep(const void* src, int S, int ld, int T, int f32, void* cq, int ldq, void* cache, int dq,
                                 int nq, int dkv, int nkv, int dkr, int rot, int rank8, int row, const float* qw,
                                 const float* kvw, float eps, const void* cs, const int* positions, const int* seq_idx,
-                                const int* block_tables, int bt_stride, int page, hipStream_t s) {
+                                const int* block_tables, int bt_stride, int page, int g_at, int g_n, void* g_out,
+                                int g_ldo, hipStream_t s) {
     if (T <= 0) return 0;
+    const GeluJob job{g_at, g_n, g_ldo, g_out};
+    if (!gelu_job_ok(job, S, ld)) return (int)hipErrorInvalidValue;
     if (nq <= 0 || dq % 8 || ld % 8 || ldq % 8 || ldq < (nq + 7) / 8 * 8 || (f32 && S < 1) || page <= 0 ||
         (dkv >= 0 && (nkv <= 0 || dkv % 8 || rot % 2 || rank8 < nkv || rank8 % 8 || row < rank8 + rot || row % 8)))
         return (int)hipErrorInvalidValue;
     const PrepArgs a{dq, nq, ldq, dkv, nkv, dkr, rot, rank8, row, qw, kvw, eps, (const float2*)cs, positions, seq_idx,
                      block_tables, bt_stride, page};
     const ProjSrc p{src, S, (size_t)T * ld, ld};
-    if (f32) return launch_prep<true, float>(p, a, cq, cache, T, s);
-    if (S) return launch_prep<true, bf16>(p, a, cq, cache, T, s);
-    return launch_prep<false, bf16>(p, a, cq, cache, T, s);
+    if (f32) return launch_prep<true, float>(p, a, cq, cache, T, job, s);
+    if (S) return launch_prep<true, bf16>(p, a, cq, cache, T, job, s);
+    return launch_prep<false, bf16>(p, a, cq, cache, T, job, s);
 }
 
 // ------------------------------------------------------------------------------------------------ per-head products

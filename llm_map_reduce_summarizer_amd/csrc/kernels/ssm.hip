@@ -96,8 +96,15 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ProjSrc src, int at, con
 template <bool PARTS, typename T, int TAPS>
 __global__ __launch_bounds__(64) void conv_step_kernel(ProjSrc src, int at, const float* __restrict__ kernel,
                                                        const float* __restrict__ bias, float* __restrict__ state,
-                                                       SegArgs sg, T* __restrict__ out, int C) {
+                                                       SegArgs sg, T* __restrict__ out, int C, GeluJob job) {
     const int t = blockIdx.y, c = 4 * (blockIdx.x * 64 + threadIdx.x);
+    if constexpr (PARTS) {
+        const int own = (C + 255) / 256;
+        if ((int)blockIdx.x >= own) {
+            gelu_piece<true, T>(src, job, t, 8 * (((int)blockIdx.x - own) * 64 + threadIdx.x));
+            return;
+        }
+    }
     if (c >= C) return;
     const bool cont = sg.pos0[t] > 0;
     float* st = state + (size_t)sg.slots[t] * (TAPS - 1) * C + c;
@@ -184,12 +191,13 @@ __global__ __launch_bounds__(256) void conv_state_kernel(ProjSrc src, int at, fl
 
 template <bool PARTS, typename T>
 static void launch_conv(const ProjSrc& p, int at, const float* kernel, const float* bias, float* state,
-                        const SegArgs& sg, void* out, int T_, int nseg, int C, int taps, hipStream_t s) {
+                        const SegArgs& sg, void* out, int T_, int nseg, int C, int taps, const GeluJob& job,
+                        hipStream_t s) {
     const int blocks = (int)(((long long)T_ * (C / 8) + 255) / 256);
     constexpr int RUN = 8;
     if (!sg.cu) {
-        const dim3 g(ceil_div(C / 4, 64), T_);
-#define STEP_T(TP) conv_step_kernel<PARTS, T, TP><<<g, 64, 0, s>>>(p, at, kernel, bias, state, sg, (T*)out, C)
+        const dim3 g(ceil_div(C / 4, 64) + ceil_div(job.n, 512), T_);
+#define STEP_T(TP) conv_step_kernel<PARTS, T, TP><<<g, 64, 0, s>>>(p, at, kernel, bias, state, sg, (T*)out, C, job)
         if (taps == 4) STEP_T(4);
         else if (taps == 3) STEP_T(3);
         else if (taps == 2) STEP_T(2);
@@ -209,19 +217,30 @@ static void launch_conv(const ProjSrc& p, int at, const float* kernel, const flo
         conv_state_kernel<PARTS, T><<<dim3(ceil_div(C / 8, 256), nseg), 256, 0, s>>>(p, at, state, sg, C, taps);
 }
 
-// src as ProjSrc (S = 0: bf16 rows); kernel [taps][C], bias [C], state [slots][taps - 1][C]; out [T][C] bf16 or fp32
+MRSUM_API int mrsum_gelu_cols(const void* src, int S, int ld, int T, int at, int n, void* out, int out32, int ldo,
+                              hipStream_t s);
+
+// g_n > 0: columns of the slabs through gelu besides (GeluJob).  src as ProjSrc (S = 0: bf16 rows); kernel [taps][C], bias [C], state [slots][taps - 1][C]; out [T][C] bf16 or fp32
 MRSUM_API int mrsum_conv_silu(const void* src, int S, int ld, int T, int at, const float* kernel, const float* bias,
                               float* state, const int* cu, const int* row_seg, const int* slots, const int* pos0,
-                              int nseg, void* out, int out32, int C, int taps, hipStream_t s) {
+                              int nseg, void* out, int out32, int C, int taps, int g_at, int g_n, void* g_out, int g_ldo,
+                              hipStream_t s) {
     if (T <= 0) return 0;
     if (C % 8 || at % 8 || ld % 8 || taps < 1 || at + C > ld || (cu && !row_seg) || (!cu && (nseg != T || T > 65535)) ||
         (out32 && S < 1) || nseg > 65535)
         return (int)hipErrorInvalidValue;
     const ProjSrc p{src, S, (size_t)T * ld, ld};
     const SegArgs sg{cu, row_seg, slots, pos0};
-    if (out32) launch_conv<true, float>(p, at, kernel, bias, state, sg, out, T, nseg, C, taps, s);
-    else if (S) launch_conv<true, bf16>(p, at, kernel, bias, state, sg, out, T, nseg, C, taps, s);
-    else launch_conv<false, bf16>(p, at, kernel, bias, state, sg, out, T, nseg, C, taps, s);
+    GeluJob job{g_at, g_n, g_ldo, g_out};
+    if (!gelu_job_ok(job, S, ld)) return (int)hipErrorInvalidValue;
+    if (job.n && (cu || taps < 2 || taps > 4)) {  // only the step form takes it along
+        const int e = mrsum_gelu_cols(src, S, ld, T, g_at, g_n, g_out, out32, g_ldo, s);
+        if (e) return e;
+        job.n = 0;
+    }
+    if (out32) launch_conv<true, float>(p, at, kernel, bias, state, sg, out, T, nseg, C, taps, job, s);
+    else if (S) launch_conv<true, bf16>(p, at, kernel, bias, state, sg, out, T, nseg, C, taps, job, s);
+    else launch_conv<false, bf16>(p, at, kernel, bias, state, sg, out, T, nseg, C, taps, job, s);
     return (int)hipGetLastError();
 }
 

@@ -209,13 +209,20 @@ class HybridModel:
     def _mix(self, i: int, la: HybridLayer, x: torch.Tensor, b, kv) -> torch.Tensor:
         a = torch.empty(x.shape[0], la.k_out, dtype=self.dtype, device=self.device)
         if la.ff:
-            u = ops.project_gelu(x, la.w.w_in, la.n_mix, a, la.ff_col, la.ff)
+            u, gelu = ops.project_gelu(x, la.w.w_in, la.n_mix, a, la.ff_col, la.ff)
         else:
+            gelu = None
             u = ops.project(x, la.w.w_in, "qkv")
             if la.ssm is None and la.k_mix < la.k_out:
                 a[:, la.k_mix:].zero_()
         for m in la.mixers:
-            m.run(i, u, a, b, kv, self.cfg.rms_eps)
+            if gelu is not None and m.takes_gelu:
+                m.run(i, u, a, b, kv, self.cfg.rms_eps, gelu)
+                gelu = None
+            else:
+                m.run(i, u, a, b, kv, self.cfg.rms_eps)
+        if gelu is not None:
+            ops.gelu_cols(u, gelu)
         return ops.project(a, la.w.w_o, "o")
 
     def _forward(self, b, kv) -> torch.Tensor:

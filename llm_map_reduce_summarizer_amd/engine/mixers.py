@@ -6,7 +6,8 @@ A mixer owns a range of columns of its layer's fused input projection and of its
     columns(take)      reserve projection columns; ``width`` is what it writes into the joint output rows
     load(...)          its weights, asked for by checkpoint name
     cache_shape / state_shape     what a sequence holds for it: paged rows, recurrent state
-    run(i, u, a, b, kv, eps)      projection rows u -> a[:, col : col + width]
+    run(i, u, a, b, kv, eps, gelu)      projection rows u -> a[:, col : col + width]; ``gelu``: the layer's pending
+                                  feed-forward columns (ops.project_gelu), for mixers that take them along (takes_gelu)
 
 ``b`` is the batch: ``n_decode`` leading single tokens (decode kernels), prompt portions behind them.
 """
@@ -51,6 +52,7 @@ class Mixer:
     width = 0          # columns of the joint output rows
     col = 0            # first of them
     scale = 1.0        # factor on this mixer's share of the layer's sum
+    takes_gelu = False
 
     def __init__(self):
         self.w = SimpleNamespace()
@@ -122,7 +124,7 @@ class AttnMixer(Mixer):
         r = self.spec.heads // self.spec.kv_heads
         return r, lambda: ops.prefill_items(lens, r)
 
-    def run(self, i, u, a, b, kv, eps) -> None:
+    def run(self, i, u, a, b, kv, eps, gelu=None) -> None:
         sp, w, page, T = self.spec, self.w, kv.page, a.shape[0]
         kc, vc = kv.k[i], kv.v[i]
         q, gate = ops.qkv_prep(u, self, w.qkv_bias, w.q_norm, w.k_norm, eps, self.scale, b.positions, b.seq_idx,
@@ -144,6 +146,8 @@ class AttnMixer(Mixer):
 
 class SSMMixer(Mixer):
     """Mamba-2 (SSMSpec)."""
+
+    takes_gelu = True
 
     def __init__(self, spec: SSMSpec, device: torch.device, dtype: torch.dtype, scale: float):
         super().__init__()
@@ -175,9 +179,9 @@ class SSMMixer(Mixer):
         s = self.spec
         return (up(s.channels, 8), s.conv, s.heads, s.vdim, s.state)
 
-    def run(self, i, u, a, b, kv, eps) -> None:
+    def run(self, i, u, a, b, kv, eps, gelu=None) -> None:
         s, w, st = self.spec, self.w, kv.state
-        xbc = ops.conv_silu(u, self.xbc, w.conv, w.conv_b, st.conv[i], b.segs, self.dtype)
+        xbc = ops.conv_silu(u, self.xbc, w.conv, w.conv_b, st.conv[i], b.segs, self.dtype, gelu)
         y = ops.ssm_scan(xbc, u, self.dt, w.dt_bias, w.a_neg, w.d_skip, st.ssm[i], b.segs, s.heads, s.vdim, s.state,
                          s.groups)
         ops.gated_norm(y, u, self.z, w.ssm_norm, s.norm_groups, eps, self.scale, a, self.col)
@@ -190,6 +194,8 @@ class LatentMixer(Mixer):
     head's unrotated keys and values (one product), and flash attention runs on [expanded key | shared rotated part].
     Decoded tokens, 32-bit models and head sizes outside the MFMA kernels: the key expansion is absorbed into the
     query, so scores and value sums run on the cached rows themselves, and the value expansion follows."""
+
+    takes_gelu = True
 
     def __init__(self, spec: LatentSpec, device: torch.device, dtype: torch.dtype):
         super().__init__()
@@ -260,12 +266,12 @@ class LatentMixer(Mixer):
         rows = ops.latent_block_rows(self.qw, self.vp)
         return ("latent", rows), lambda: ops.latent_items(lens, rows)
 
-    def run(self, i, u, a, b, kv, eps) -> None:
+    def run(self, i, u, a, b, kv, eps, gelu=None) -> None:
         s, w, page, T = self.spec, self.w, kv.page, a.shape[0]
         src = i if s.kv_from is None else s.kv_from
         cache, cs = kv.k[src], b.rotary[s.rot]
         cq = ops.latent_prep(u, self, w.dq_norm, w.dkv_norm, eps, cs, b.positions, b.seq_idx, b.tables, cache, page,
-                             self.dtype)
+                             self.dtype, gelu)
         q = ops.project(cq, w.w_uq, "qkv")
         nd = b.n_decode if self.flash else T
         if nd:
@@ -295,6 +301,8 @@ class LatentMixer(Mixer):
 
 class DeltaMixer(Mixer):
     """Gated delta rule (DeltaSpec).  The short convolutions of q, k and v run as one over adjacent columns."""
+
+    takes_gelu = True
 
     def __init__(self, spec: DeltaSpec, device: torch.device, dtype: torch.dtype):
         super().__init__()
@@ -329,9 +337,9 @@ class DeltaMixer(Mixer):
         s = self.spec
         return (self.channels, s.conv, s.heads, s.vdim, s.dim)
 
-    def run(self, i, u, a, b, kv, eps) -> None:
+    def run(self, i, u, a, b, kv, eps, gelu=None) -> None:
         w, st = self.w, kv.state
-        x = ops.conv_silu(u, self.q, w.conv, w.conv_b, st.conv[i], b.segs, self.dtype)
+        x = ops.conv_silu(u, self.q, w.conv, w.conv_b, st.conv[i], b.segs, self.dtype, gelu)
         ops.delta_mix(x, u, self, w.a_neg, w.dt_bias, w.norm, eps, st.ssm[i], b.segs, a)
 
 

@@ -299,8 +299,8 @@ def attn_rows(q, kcache, vcache, positions, seq_idx, block_tables, hq, hkv, pitc
                               out)
 
 
-def conv_silu(u, at, kernel, bias, state, segs, dtype):
-    return _impl(u).conv_silu(u, at, kernel, bias, state, segs, dtype)
+def conv_silu(u, at, kernel, bias, state, segs, dtype, gelu=None):
+    return _impl(u).conv_silu(u, at, kernel, bias, state, segs, dtype, gelu)
 
 
 def ssm_scan(xbc, u, dt_at, dt_bias, a_neg, d_skip, state, segs, heads, vdim, n_state, groups):
@@ -317,8 +317,13 @@ def embed_bigram(ids, segs, table, bigram, scale, mul_prev, mul_cur, w, eps, las
 
 
 def project_gelu(x, w, n, out, col, cols):
-    """x @ w[:n]^T in the forms of ``project``, and gelu(x @ w[n : n + cols]^T) into out[:, col : col + cols]."""
+    """(x @ w[:n]^T in the forms of ``project``, job): gelu(x @ w[n : n + cols]^T) goes into out[:, col : col + cols], at
+    once (job None) or with a later kernel that is handed the job (conv_silu, latent_prep, gelu_cols)."""
     return _impl(x).project_gelu(x, w, n, out, col, cols)
+
+
+def gelu_cols(u, job):
+    return _impl(u).gelu_cols(u, job)
 
 
 # ---------------------------------------------------------------- latent attention (``m``: engine.mixers.LatentMixer)
@@ -365,8 +370,8 @@ def latent_workspace(B, heads, rank, max_ctx, device):
     return LatentWorkspace(B, heads, rank, max_ctx, device)
 
 
-def latent_prep(u, m, dq_norm, dkv_norm, eps, cs, positions, seq_idx, block_tables, cache, page, dtype):
-    return _impl(u).latent_prep(u, m, dq_norm, dkv_norm, eps, cs, positions, seq_idx, block_tables, cache, page, dtype)
+def latent_prep(u, m, dq_norm, dkv_norm, eps, cs, positions, seq_idx, block_tables, cache, page, dtype, gelu=None):
+    return _impl(u).latent_prep(u, m, dq_norm, dkv_norm, eps, cs, positions, seq_idx, block_tables, cache, page, dtype, gelu)
 
 
 def latent_absorb(q, n, m, w_uk, cs, positions, dtype):

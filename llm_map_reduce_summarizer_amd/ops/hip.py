@@ -11,7 +11,7 @@ from __future__ import annotations
 
 import ctypes
 import os
-from typing import Optional
+from typing import NamedTuple, Optional
 
 import torch
 
@@ -68,7 +68,7 @@ _SIGS = {
                         _vp, _vp, _c_int, _c_int, _vp],
     "mrsum_gemm32": [_vp, _c_int, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp],
     "mrsum_conv_silu": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int,
-                        _c_int, _c_int, _vp],
+                        _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _vp],
     "mrsum_ssm_step": [_vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
                        _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp],
     "mrsum_ssm_chunk": [_vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _vp,
@@ -79,7 +79,7 @@ _SIGS = {
                            _c_int, _c_int, _c_float, _c_float, _vp],
     "mrsum_gelu_cols": [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _vp],
     "mrsum_latent_prep": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _vp] + [_c_int] * 8 +
-                         [_vp, _vp, _c_float, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp],
+                         [_vp, _vp, _c_float, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _vp],
     "mrsum_head_product": [_vp] + [_c_int] * 6 + [_vp, _c_int, _c_int, _vp] + [_c_int] * 8 + [_vp, _vp, _vp, _vp, _c_int, _vp],
     "mrsum_latent_rope": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp],
     "mrsum_latent_gather": [_vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _vp, _vp],
@@ -1619,7 +1619,7 @@ def attn_rows(q, kcache, vcache, positions, seq_idx, block_tables, hq: int, hkv:
                                   out.stride(0), 1 if dt == torch.float32 else 0, _stream()), "attn_rows")
 
 
-def conv_silu(u, at: int, kernel, bias, state, segs, dtype) -> torch.Tensor:
+def conv_silu(u, at: int, kernel, bias, state, segs, dtype, gelu=None) -> torch.Tensor:
     ptr, S, ld, T = _src(u, dtype, "conv_silu")
     _f32(kernel, bias, state)
     taps, C = kernel.shape
@@ -1629,7 +1629,7 @@ def conv_silu(u, at: int, kernel, bias, state, segs, dtype) -> torch.Tensor:
     out = torch.empty(T, C, dtype=dtype, device=u.device)
     _check(_fn("mrsum_conv_silu")(ptr, S, ld, T, at, _p(kernel), _p(bias), _p(state), cu, row_seg, _p(segs.slots),
                                   _p(segs.pos0), segs.n, _p(out), 1 if dtype == torch.float32 else 0, C, taps,
-                                  _stream()), "conv_silu")
+                                  *_gelu_args(gelu, T, ld, dtype), _stream()), "conv_silu")
     return out
 
 
@@ -1730,31 +1730,46 @@ def embed_bigram(ids, segs, table, bigram, scale: float, mul_prev: int, mul_cur:
     return out
 
 
-def gelu_cols(u, at: int, n: int, out, col: int) -> None:
-    """out[:, col : col + n] = gelu of columns [at, at + n) of fp32 slabs ``u``."""
-    ptr, S, ld, T = _src(u, torch.bfloat16, "gelu_cols")
-    _req(S >= 1 and at + n <= ld and out.stride(1) == 1 and out.shape[0] == T and col % 8 == 0 and col + n <= out.shape[1]
-         and out.stride(0) % 8 == 0 and out.dtype in (torch.bfloat16, torch.float32), "gelu_cols: shapes")
-    es = out.element_size()
-    _check(_fn("mrsum_gelu_cols")(ptr, S, ld, T, at, n, out.data_ptr() + es * col, 1 if es == 4 else 0, out.stride(0),
-                                  _stream()), "gelu_cols")
+class GeluCols(NamedTuple):
+    """A pending job on the slabs of project_gelu: out[:, col : col + n] = gelu of columns [at, at + n).  Done by gelu_cols,
+    or taken along by the kernel that reads the same slabs next (conv_silu, latent_prep)."""
+    at: int
+    n: int
+    out: torch.Tensor
+    col: int
+
+
+def _gelu_args(job: Optional[GeluCols], T: int, ld: int, dtype):
+    """(first column, columns, output, row stride) of the kernels' GeluJob, checked."""
+    if job is None:
+        return 0, 0, None, 0
+    out = job.out
+    _req(job.at + job.n <= ld and out.is_cuda and out.stride(1) == 1 and out.shape[0] == T and job.col % 8 == 0
+         and job.col + job.n <= out.shape[1] and out.dtype == dtype and out.data_ptr() % 16 == 0, "gelu columns: shapes")
+    return job.at, job.n, out.data_ptr() + out.element_size() * job.col, out.stride(0)
+
+
+def gelu_cols(u, job: GeluCols) -> None:
+    ptr, S, ld, T = _src(u, job.out.dtype, "gelu_cols")
+    at, n, out, ldo = _gelu_args(job, T, ld, job.out.dtype)
+    _check(_fn("mrsum_gelu_cols")(ptr, S, ld, T, at, n, out, 1 if job.out.dtype == torch.float32 else 0, ldo, _stream()),
+           "gelu_cols")
 
 
 def project_gelu(x, w, n: int, out, col: int, cols: int):
-    """Decode row counts and 32-bit mode: one product of all rows of ``w`` whose gelu columns are summed from its slabs.
-    More rows: two MFMA GEMMs, the second with the gelu in its epilogue, straight into ``out``."""
+    """Decode row counts and 32-bit mode: one product of all rows of ``w``; its gelu columns are a pending GeluCols job.
+    More rows: two MFMA GEMMs, the second with the gelu in its epilogue, straight into ``out``, and no job."""
     M = x.shape[0]
     _req(n % 8 == 0 and n + cols <= w.shape[0], "project_gelu: rows")
     if x.dtype == torch.bfloat16 and M > STREAM_MAX_M:
         gemm(x, w[n: n + cols], out=out[:, col: col + cols], gelu=True)
-        return gemm(x, w[:n])
+        return gemm(x, w[:n]), None
     from . import project
     u = project(x, w, "qkv")
-    if u.dim() == 2:  # a shape only the GEMM takes
-        gemm(x, w[n: n + cols], out=out[:, col: col + cols], gelu=True)
-    else:
-        gelu_cols(u, n, cols, out, col)
-    return u
+    if u.dim() == 3:
+        return u, GeluCols(n, cols, out, col)
+    gemm(x, w[n: n + cols], out=out[:, col: col + cols], gelu=True)  # a shape only the GEMM takes
+    return u, None
 
 
 # ------------------------------------------------------------------ latent attention (``m``: engine.mixers.LatentMixer)
@@ -1798,7 +1813,8 @@ def _rotary_ok(cs, rot: int, positions, n: int, what: str) -> None:
          and positions.numel() >= n, what + ": rotation table / positions")
 
 
-def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, block_tables, cache, page: int, dtype):
+def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, block_tables, cache, page: int, dtype,
+                gelu=None):
     sp = m.spec
     ptr, S, ld, T = _src(u, dtype, "latent_prep")
     _i32(seq_idx, block_tables)
@@ -1816,7 +1832,7 @@ def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, blo
                                     _p(cache) if own else None, m.dq, sp.q_rank, m.dkv if own else -1, sp.kv_rank,
                                     m.dkr if own else 0, sp.rot_dim, m.rank8, m.row, _p(dq_norm), _p(dkv_norm), eps, _p(cs),
                                     _p(positions), _p(seq_idx), _p(block_tables), block_tables.stride(0), page,
-                                    _stream()), "latent_prep")
+                                    *_gelu_args(gelu, T, ld, dtype), _stream()), "latent_prep")
     return out
 
 

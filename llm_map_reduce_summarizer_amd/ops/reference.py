@@ -490,7 +490,7 @@ def attn_rows(q, kcache, vcache, positions, seq_idx, block_tables, hq: int, hkv:
         out[t, : hq * pitch] = o[:, :pitch].reshape(-1).to(out.dtype)
 
 
-def conv_silu(u, at: int, kernel, bias, state, segs, dtype) -> torch.Tensor:
+def conv_silu(u, at: int, kernel, bias, state, segs, dtype, gelu=None) -> torch.Tensor:
     """silu(causal per-channel convolution) of columns [at, at + C) of ``u``; ``kernel`` [taps, C] (last tap = current
     token), ``state`` [slots, taps - 1, C] the inputs before each segment (oldest first), updated in place."""
     taps, C = kernel.shape
@@ -556,11 +556,11 @@ def embed_bigram(ids, segs, table, bigram, scale: float, mul_prev: int, mul_cur:
     return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w
 
 
-def project_gelu(x, w, n: int, out, col: int, cols: int) -> torch.Tensor:
+def project_gelu(x, w, n: int, out, col: int, cols: int):
     """The first ``n`` rows of ``w`` as project(); gelu of the next ``cols`` into out[:, col : col + cols]."""
     u = x.float() @ w[: n + cols].float().t()
     out[:, col: col + cols] = torch.nn.functional.gelu(u[:, n:], approximate="tanh").to(out.dtype)
-    return u[None, :, :n].contiguous()
+    return u[None, :, :n].contiguous(), None
 
 
 def yarn_inv_freq(dims: int, base: float, yarn=None) -> torch.Tensor:
@@ -593,7 +593,8 @@ def rotate_half(x: torch.Tensor, cs: torch.Tensor) -> torch.Tensor:
 
 
 # ----------------------------------------------------------------- latent attention (``m``: engine.mixers.LatentMixer)
-def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, block_tables, cache, page: int, dtype):
+def latent_prep(u, m, dq_norm, dkv_norm, eps: float, cs, positions, seq_idx, block_tables, cache, page: int, dtype,
+                gelu=None):
     """Normed query latents [T, m.cq] (zero-padded); for a layer with its own latents, the row [normed latent | rotated
     key part] of every token into the paged cache."""
     sp, r = m.spec, rows32(u)
