@@ -24,6 +24,13 @@ __device__ __forceinline__ bf16x8 tr8(const bf16* lo, const bf16* hi) {
     const s4 b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s4*)hi);
     return __builtin_bit_cast(bf16x8, (s8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]}));
 }
+// maximum over the four 16-lane groups
+__device__ __forceinline__ float groups_max(float v) {
+    const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    v = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
+    const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
+}
 __device__ __forceinline__ float halves(float v, bool max) {
     const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
     const float a = __uint_as_float(r[0]), b = __uint_as_float(r[1]);
@@ -271,6 +278,18 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
     const int sp = blockIdx.x, h0 = DH * blockIdx.y, b = blockIdx.z;
     const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4, q4 = r16 >> 2, p4 = 4 * (r16 & 3);
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6), kb4 = w & 3, hb = w >> 2;
+    bf16x8 qf[KB];  // this wave's 16 heads
+    {
+        const int h = h0 + 16 * hb + r16;
+        const bf16* qp = a.q + ((size_t)b * a.H + min(h, a.H - 1)) * a.row;
+#pragma unroll
+        for (int kb = 0; kb < KB; ++kb) {
+            const int c = 32 * kb + 8 * g;
+            u32x4 v = *reinterpret_cast<const u32x4*>(qp + min(c, a.row - 8));
+            if (c >= a.row || h >= a.H) v = u32x4{0, 0, 0, 0};
+            qf[kb] = as8(v);
+        }
+    }
     const int pos = a.positions[b], pages = pos / BN + 1;
     const int used = min(a.S, pages);  // splits past them are empty
     const int p0 = sp < used ? (int)((long long)pages * sp / used) : 0;
@@ -284,9 +303,12 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
         const int c = min(tid + 512 * i, total - 1);
         at[i] = c / rc * LK + 8 * (c % rc);
     }
+    // the id of the page after the one being fetched is read ahead, so that fetching never waits for it
+    int id = 0;
 #define LOAD_PAGE(p)                                                                                    \
     {                                                                                                   \
-        const bf16* pg_ = a.cache + (size_t)bt[p] * BN * a.row;                                         \
+        const bf16* pg_ = a.cache + (size_t)id * BN * a.row;                                            \
+        id = bt[min((p) + 1, p1 - 1)];                                                                  \
         _Pragma("unroll") for (int i = 0; i < IT; ++i)                                                  \
             reg[i] = *reinterpret_cast<const u32x4*>(pg_ + 8 * min(tid + 512 * i, total - 1));          \
     }
@@ -295,21 +317,10 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
 #pragma unroll
     for (int vb = 0; vb < VB; ++vb) acc[vb][0] = acc[vb][1] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (p0 < p1) {
+        id = bt[p0];
         LOAD_PAGE(p0)
-        bf16x8 qf[KB];  // this wave's 16 heads
-        {
-            const int h = h0 + 16 * hb + r16;
-            const bf16* qp = a.q + ((size_t)b * a.H + min(h, a.H - 1)) * a.row;
-#pragma unroll
-            for (int kb = 0; kb < KB; ++kb) {
-                const int c = 32 * kb + 8 * g;
-                u32x4 v = *reinterpret_cast<const u32x4*>(qp + min(c, a.row - 8));
-                if (c >= a.row || h >= a.H) v = u32x4{0, 0, 0, 0};
-                qf[kb] = as8(v);
-            }
-        }
         // columns past the row: zeros in both stages
-        const int rz = 4 * KB + 1 - rc;
+        const int rz = 4 * KB - rc;
         for (int i = tid; i < 2 * BN * rz; i += 512)
             *reinterpret_cast<u32x4*>(&sk[0][0] + (i / rz) * LK + 8 * (rc + i % rz)) = u32x4{0, 0, 0, 0};
 #pragma unroll
@@ -338,8 +349,7 @@ __global__ __launch_bounds__(512, 1) void latent_decode_kernel(const LatDecode a
                 s[j] = j <= kmax ? s[j] * a.scale_log2 : -INFINITY;
                 mx = fmaxf(mx, s[j]);
             }
-            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            mx = groups_max(mx);
             if (g == 0) smax[16 * hb + r16][kb4] = mx;
             __syncthreads();
             float alpha[2];
