@@ -36,6 +36,9 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x,
     const float an = a.a_neg[head], db = a.dt_bias[head];
     for (int t = b; t < e; ++t) {
         const T* row = x + (size_t)t * a.ldx;
+        // this thread's output column: gate and weight are read before they are needed
+        const int p0 = min(tid, a.P - 1);
+        const float z0 = proj_at<PARTS>(a.u, t, a.g_at + head * a.P + p0), w0 = a.norm[p0];
         float q[NV][4], k[NV][4];
         float qq = 0.f, kk = 0.f, kq = 0.f;
 #pragma unroll
@@ -102,8 +105,8 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x,
         const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.P + a.eps);
         T* o = out + (size_t)t * a.ldo + a.col + head * a.P;
         for (int p = tid; p < a.P; p += NT) {
-            const float z = proj_at<PARTS>(a.u, t, a.g_at + head * a.P + p);
-            o[p] = (T)(s_o[p] * inv * a.norm[p] * z * logistic_for<T>(z));
+            const float z = p < NT ? z0 : proj_at<PARTS>(a.u, t, a.g_at + head * a.P + p);
+            o[p] = (T)(s_o[p] * inv * (p < NT ? w0 : a.norm[p]) * z * logistic_for<T>(z));
         }
         if (head == 0)
             for (int c = a.heads * a.P + tid; c < a.width; c += NT) out[(size_t)t * a.ldo + a.col + c] = (T)0.f;

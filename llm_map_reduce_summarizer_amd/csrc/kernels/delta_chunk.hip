@@ -29,10 +29,6 @@ __device__ __forceinline__ s4 tr4(const bf16* p) { return __builtin_amdgcn_ds_re
 __device__ __forceinline__ bf16x8 join(s4 a, s4 b) {
     return __builtin_bit_cast(bf16x8, (s8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]}));
 }
-// columns [0, 4) and [16, 20) of a row: an operand in the order of two accumulator tiles
-__device__ __forceinline__ bf16x8 pair4(const bf16* p) {
-    return join(*reinterpret_cast<const s4*>(p), *reinterpret_cast<const s4*>(p + 16));
-}
 __device__ __forceinline__ f32x4 mma(bf16x8 a, bf16x8 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
@@ -40,15 +36,37 @@ __device__ __forceinline__ f32x4 mma32(float a, float b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 __device__ __forceinline__ void split(f32x4 a, f32x4 b, bf16x8& hi, bf16x8& lo) {
+    u32x4 h, l;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-        hi[j] = (bf16)a[j];
-        lo[j] = (bf16)(a[j] - (float)hi[j]);
-        hi[4 + j] = (bf16)b[j];
-        lo[4 + j] = (bf16)(b[j] - (float)hi[4 + j]);
+        const float x = j < 2 ? a[2 * j] : b[2 * j - 4], y = j < 2 ? a[2 * j + 1] : b[2 * j - 3];
+        h[j] = pack2(x, y);
+        l[j] = pack2(x - __uint_as_float(h[j] << 16), y - __uint_as_float(h[j] & 0xffff0000u));
     }
+    hi = __builtin_bit_cast(bf16x8, h);
+    lo = __builtin_bit_cast(bf16x8, l);
 }
 __device__ __forceinline__ int frag_of(int ib, int jp) { return ib < 2 ? ib : 2 * (ib - 1) + jp; }
+
+// c += L b for a lower-triangular 64 x 64 L given as operand tiles (hi, then lo), b as operands (hi, lo) or as four
+// accumulator tiles
+__device__ __forceinline__ void lower(f32x4* c, const uint4* l, const bf16x8* hi, const bf16x8* lo) {
+#pragma unroll
+    for (int jp = 0; jp < 2; ++jp) {
+#pragma unroll
+        for (int ib = 2 * jp; ib < 4; ++ib) c[ib] = mma(__builtin_bit_cast(bf16x8, l[frag_of(ib, jp)]), hi[jp], c[ib]);
+#pragma unroll
+        for (int ib = 2 * jp; ib < 4; ++ib) c[ib] = mma(__builtin_bit_cast(bf16x8, l[frag_of(ib, jp)]), lo[jp], c[ib]);
+#pragma unroll
+        for (int ib = 2 * jp; ib < 4; ++ib) c[ib] = mma(__builtin_bit_cast(bf16x8, l[FR + frag_of(ib, jp)]), hi[jp], c[ib]);
+    }
+}
+__device__ __forceinline__ void lower(f32x4* c, const uint4* l, const f32x4* b) {
+    bf16x8 hi[2], lo[2];
+    split(b[0], b[1], hi[0], lo[0]);
+    split(b[2], b[3], hi[1], lo[1]);
+    lower(c, l, hi, lo);
+}
 }  // namespace
 
 // x: convolved rows.  chunks: (first row, end row) of every chunk.  Per (chunk, head): frags [FRAGS] 16-byte pieces,
@@ -70,6 +88,15 @@ __global__ __launch_bounds__(256, NB <= 4 ? 4 : 2) void delta_prep_kernel(const 
     const int2 ch = chunks[ck];
     const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4;
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    // raw decays and step sizes of a head's 64 tokens (wave 0), fetched a head ahead
+    float ar = 0.f, br = 0.f;
+    const int rep = a.heads / a.kv_heads, tok = min(ch.x + lane, ch.y - 1);
+#define LOAD_RAW(HEAD)                                                                                          \
+    if (w == 0) {                                                                                               \
+        ar = a.u.S ? proj_at<true>(a.u, tok, a.a_at + (HEAD)) : proj_at<false>(a.u, tok, a.a_at + (HEAD));      \
+        br = a.u.S ? proj_at<true>(a.u, tok, a.b_at + (HEAD)) : proj_at<false>(a.u, tok, a.b_at + (HEAD));      \
+    }
+    LOAD_RAW(kh * rep)
     for (int i = tid; i < Q * 4 * NB; i += 256) {
         const int row = i / (4 * NB), n = 8 * (i % (4 * NB)), t = ch.x + row;
         u32x4 k = {0, 0, 0, 0}, q = {0, 0, 0, 0};
@@ -123,7 +150,7 @@ __global__ __launch_bounds__(256, NB <= 4 ? 4 : 2) void delta_prep_kernel(const 
             }
         }
     }
-    const int rep = a.heads / a.kv_heads, i = 16 * w + r16;
+    const int i = 16 * w + r16;
     for (int hr = 0; hr < rep; ++hr) {
         const int head = kh * rep + hr;
         __syncthreads();  // factors ready; the previous head's readers are done
@@ -131,8 +158,6 @@ __global__ __launch_bounds__(256, NB <= 4 ? 4 : 2) void delta_prep_kernel(const 
             const int t = ch.x + lane;
             float c = 0.f, beta = 0.f;
             if (t < ch.y) {
-                const float ar = a.u.S ? proj_at<true>(a.u, t, a.a_at + head) : proj_at<false>(a.u, t, a.a_at + head);
-                const float br = a.u.S ? proj_at<true>(a.u, t, a.b_at + head) : proj_at<false>(a.u, t, a.b_at + head);
                 beta = logistic(br);
                 c = a.a_neg[head] * LOG2E * softplus(ar + a.dt_bias[head]);
             }
@@ -150,6 +175,7 @@ __global__ __launch_bounds__(256, NB <= 4 ? 4 : 2) void delta_prep_kernel(const 
             v[128 + lane] = __builtin_amdgcn_exp2f(last - c) * rk;
             if (lane == 0) v[192] = __builtin_amdgcn_exp2f(last);
         }
+        if (hr + 1 < rep) LOAD_RAW(head + 1)
         __syncthreads();
         uint4* fr = frags + ((size_t)ck * a.heads + head) * FRAGS;
         const float ci = s_c[i], bi = s_beta[i] * s_rk[i], qi = s_rq[i];
@@ -255,7 +281,93 @@ __global__ __launch_bounds__(256, NB <= 4 ? 4 : 2) void delta_prep_kernel(const 
     }
 }
 
-// Grid (blocks of 16 WPB value columns, heads, segments).  segs: (segment, first row, end row, first chunk).
+#undef LOAD_RAW
+
+// Rows of k and q in LDS.  128 and 256 wide: unpadded, 16-byte pieces exchanged by a row-dependent mask, so that the 16 rows
+// of a read lie in different banks; narrower: padded to the same end.
+template <int NB>
+constexpr int row_stride() { return NB >= 4 ? 32 * NB : 32 * NB + 8; }
+template <int NB>
+__device__ __forceinline__ int row_at(int row, int col) {
+    if constexpr (NB >= 4) return row * 32 * NB + (col ^ ((((row & 3) << 2) | ((row >> 2) & 3)) << 3));
+    return row * row_stride<NB>() + col;
+}
+// Rows 4 g + e of state tile nb are this dimension plus e: the tiles of a pair take turns in fours, so that a lane's operand
+// of the products over the state is eight neighbouring columns of a row.
+__device__ __forceinline__ int tile_row(int nb, int g) { return 32 * (nb >> 1) + 8 * g + 4 * (nb & 1); }
+
+// Staging of a chunk through the registers of NTH threads.  Loads are unconditional, so that later waits can count them: rows
+// past the segment and columns past the head repeat valid ones, and are zeroed on the way into LDS.  Addresses are a uniform
+// base and a 32-bit offset.
+#define LOAD_CHUNK(T0, CK)                                                                                  \
+    {                                                                                                       \
+        const size_t row0_ = (size_t)(T0) * a.ldx;                                                          \
+        const int last_ = re - 1 - (T0);                                                                    \
+        _Pragma("unroll") for (int i = 0; i < KIT; ++i) {                                                   \
+            const int idx = tid + NTH * i, n = min(8 * (idx % (4 * NB)), a.N - 8);                          \
+            const uint32_t at_ = 2u * (uint32_t)(min(idx / (4 * NB), last_) * a.ldx + n);                   \
+            kreg[i] = *reinterpret_cast<const u32x4*>(reinterpret_cast<const char*>(kcol + row0_) + at_);   \
+            qreg[i] = *reinterpret_cast<const u32x4*>(reinterpret_cast<const char*>(qcol + row0_) + at_);   \
+        }                                                                                                   \
+        _Pragma("unroll") for (int i = 0; i < VR; ++i) {                                                     \
+            const int idx = tid + NTH * i, c = min(8 * (idx % (2 * WPB)), a.P - 8 - pb);                    \
+            const uint32_t at_ = 2u * (uint32_t)(min(idx / (2 * WPB), last_) * a.ldx + c);                  \
+            vreg[i] = *reinterpret_cast<const u32x4*>(reinterpret_cast<const char*>(vcol + row0_) + at_);   \
+        }                                                                                                   \
+        const float* vs_ = vec + ((size_t)(CK) * a.heads + head) * 256;                                     \
+        _Pragma("unroll") for (int i = 0; i < VIT; ++i) vecr[i] = vs_[min(tid + NTH * i, 192)];             \
+    }
+#define STORE_CHUNK(T0)                                                                                     \
+    {                                                                                                       \
+        if ((T0) + Q > re || a.N < NN || pb + 16 * WPB > a.P) {                                             \
+            const u32x4 zero = {0, 0, 0, 0};                                                                \
+            _Pragma("unroll") for (int i = 0; i < KIT; ++i) {                                               \
+                const int idx = tid + NTH * i;                                                              \
+                const bool on = (T0) + idx / (4 * NB) < re && 8 * (idx % (4 * NB)) < a.N;                   \
+                kreg[i] = on ? kreg[i] : zero;                                                              \
+                qreg[i] = on ? qreg[i] : zero;                                                              \
+            }                                                                                               \
+            _Pragma("unroll") for (int i = 0; i < VR; ++i) {                                                 \
+                const int idx = tid + NTH * i;                                                              \
+                const bool on = (T0) + idx / (2 * WPB) < re && pb + 8 * (idx % (2 * WPB)) < a.P;            \
+                vreg[i] = on ? vreg[i] : zero;                                                              \
+            }                                                                                               \
+        }                                                                                                   \
+        _Pragma("unroll") for (int i = 0; i < KIT; ++i) {                                                   \
+            const int idx = tid + NTH * i, o_ = row_at<NB>(idx / (4 * NB), 8 * (idx % (4 * NB)));           \
+            if (KIT * NTH == Q * 4 * NB || idx < Q * 4 * NB) {                                              \
+                *reinterpret_cast<u32x4*>(sK + o_) = kreg[i];                                               \
+                *reinterpret_cast<u32x4*>(sQ + o_) = qreg[i];                                               \
+            }                                                                                               \
+        }                                                                                                   \
+        _Pragma("unroll") for (int i = 0; i < VR; ++i) {                                                     \
+            const int idx = tid + NTH * i;                                                                  \
+            *reinterpret_cast<u32x4*>(sV + idx / (2 * WPB) * LV + 8 * (idx % (2 * WPB))) = vreg[i];         \
+        }                                                                                                   \
+        _Pragma("unroll") for (int i = 0; i < VIT; ++i)                                                     \
+            if (NTH <= 256 || tid + NTH * i < 256) s_vec[tid + NTH * i] = vecr[i];                          \
+    }
+
+// o: output tiles of the chunk at t0
+#define STORE_ROWS(o)                    \
+    if (p < a.P) {                                                                                          \
+        float* yb = y + (size_t)(t0 - y0) * inner + head * a.P;                                             \
+        const uint32_t yo = 4u * (uint32_t)(4 * g * inner + p);                                             \
+        const int left = re - t0 - 4 * g;                                                                   \
+        if (t0 + Q <= re) {                                                                                 \
+            _Pragma("unroll") for (int ib = 0; ib < 4; ++ib)                                                \
+                _Pragma("unroll") for (int e = 0; e < 4; ++e)                                               \
+                    *reinterpret_cast<float*>(reinterpret_cast<char*>(yb + (size_t)(16 * ib + e) * inner) + yo) = o[ib][e];\
+        } else {                                                                                            \
+            _Pragma("unroll") for (int ib = 0; ib < 4; ++ib)                                                \
+                _Pragma("unroll") for (int e = 0; e < 4; ++e)                                               \
+                    if (16 * ib + e < left)                                                                 \
+                        *reinterpret_cast<float*>(reinterpret_cast<char*>(yb + (size_t)(16 * ib + e) * inner) + yo) = o[ib][e];\
+        }                                                                                                   \
+    }
+
+// Grid (heads, blocks of 16 WPB value columns, segments): heads first, so that the blocks of a head, which read the same
+// operands, share an XCD's L2.  segs: (segment, first row, end row, first chunk).
 template <int NB, int WPB>
 __global__ __launch_bounds__(64 * WPB, 1) void delta_chunk_kernel(const bf16* __restrict__ x, DeltaArgs a,
                                                                   const int4* __restrict__ segs,
@@ -265,14 +377,14 @@ __global__ __launch_bounds__(64 * WPB, 1) void delta_chunk_kernel(const bf16* __
                                                                   const float* __restrict__ vec,
                                                                   float* __restrict__ state, float* __restrict__ y,
                                                                   int y0) {
-    constexpr int NTH = 64 * WPB, NN = 32 * NB, LK = NN + 16, LV = 16 * WPB + 16, NT = 2 * NB;
-    constexpr int KIT = (Q * 4 * NB + NTH - 1) / NTH;  // staging rounds of k and of q (v: 2)
+    constexpr int NTH = 64 * WPB, NN = 32 * NB, LK = row_stride<NB>(), LV = 16 * WPB + 16, NT = 2 * NB, GN = NT < 4 ? NT : 4;
+    constexpr int KIT = (Q * 4 * NB + NTH - 1) / NTH, VR = 2;  // staging rounds of k and of q, of v
     constexpr int VIT = NTH < 256 ? 256 / NTH : 1;
     __shared__ __attribute__((aligned(16))) bf16 sK[Q * LK];
     __shared__ __attribute__((aligned(16))) bf16 sQ[Q * LK];
     __shared__ __attribute__((aligned(16))) bf16 sV[Q * LV];
     __shared__ __attribute__((aligned(16))) float s_vec[256];
-    const int head = blockIdx.y, pb = 16 * WPB * blockIdx.x;
+    const int head = blockIdx.x, pb = 16 * WPB * blockIdx.y;
     const int4 sg = segs[blockIdx.z];
     const int rb = sg.y, re = sg.z;
     const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4, q4 = r16 >> 2, p4 = 4 * (r16 & 3);
@@ -282,57 +394,20 @@ __global__ __launch_bounds__(64 * WPB, 1) void delta_chunk_kernel(const bf16* __
     const bf16* kcol = qcol + a.xk;
     const bf16* vcol = x + a.xv + head * a.P + pb;
     const int p = pb + 16 * w + r16;  // this lane's value column
-    u32x4 kreg[KIT], qreg[KIT], vreg[2];
+    u32x4 kreg[KIT], qreg[KIT], vreg[VR];
     float vecr[VIT];
-    // rows past the segment and columns past the head are zeros
-#define LOAD_CHUNK(T0, CK)                                                                                  \
-    {                                                                                                       \
-        _Pragma("unroll") for (int i = 0; i < KIT; ++i) {                                                   \
-            const int idx = tid + NTH * i, t = (T0) + idx / (4 * NB), n = 8 * (idx % (4 * NB));             \
-            kreg[i] = qreg[i] = u32x4{0, 0, 0, 0};                                                          \
-            if (idx < Q * 4 * NB && t < re && n < a.N) {                                                    \
-                kreg[i] = *reinterpret_cast<const u32x4*>(kcol + (size_t)t * a.ldx + n);                    \
-                qreg[i] = *reinterpret_cast<const u32x4*>(qcol + (size_t)t * a.ldx + n);                    \
-            }                                                                                               \
-        }                                                                                                   \
-        _Pragma("unroll") for (int i = 0; i < 2; ++i) {                                                     \
-            const int idx = tid + NTH * i, t = (T0) + idx / (2 * WPB), c = 8 * (idx % (2 * WPB));           \
-            vreg[i] = u32x4{0, 0, 0, 0};                                                                    \
-            if (t < re && pb + c < a.P) vreg[i] = *reinterpret_cast<const u32x4*>(vcol + (size_t)t * a.ldx + c); \
-        }                                                                                                   \
-        const float* vs_ = vec + ((size_t)(CK) * a.heads + head) * 256;                                     \
-        _Pragma("unroll") for (int i = 0; i < VIT; ++i) {                           \
-            const int idx = tid + NTH * i;                                                                  \
-            vecr[i] = idx <= 192 ? vs_[idx] : 0.f;                                                          \
-        }                                                                                                   \
-    }
-#define STORE_CHUNK()                                                                                       \
-    {                                                                                                       \
-        _Pragma("unroll") for (int i = 0; i < KIT; ++i) {                                                   \
-            const int idx = tid + NTH * i, o = idx / (4 * NB) * LK + 8 * (idx % (4 * NB));                  \
-            if (idx < Q * 4 * NB) {                                                                         \
-                *reinterpret_cast<u32x4*>(sK + o) = kreg[i];                                                \
-                *reinterpret_cast<u32x4*>(sQ + o) = qreg[i];                                                \
-            }                                                                                               \
-        }                                                                                                   \
-        _Pragma("unroll") for (int i = 0; i < 2; ++i) {                                                     \
-            const int idx = tid + NTH * i;                                                                  \
-            *reinterpret_cast<u32x4*>(sV + idx / (2 * WPB) * LV + 8 * (idx % (2 * WPB))) = vreg[i];         \
-        }                                                                                                   \
-        _Pragma("unroll") for (int i = 0; i < VIT; ++i)                             \
-            if (tid + NTH * i < 256) s_vec[tid + NTH * i] = vecr[i];                                        \
-    }
-    // state tiles: rows n = 16 nb + 4 g + e, column p
-    float* st_p = state + ((size_t)slots[sg.x] * a.heads + head) * a.P * a.N4 + (size_t)p * a.N4 + 4 * g;
+    // state tiles: rows tile_row(nb, g) + e, column p
+    float* st_p = state + ((size_t)slots[sg.x] * a.heads + head) * a.P * a.N4 + (size_t)p * a.N4;
     f32x4 st[NT];
     const bool cont = pos0[sg.x] > 0;
 #pragma unroll
     for (int nb = 0; nb < NT; ++nb) {
         st[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (cont && p < a.P && 16 * nb + 4 * g < a.N) st[nb] = *reinterpret_cast<const f32x4*>(st_p + 16 * nb);
+        const int n = tile_row(nb, g);
+        if (cont && p < a.P && n < a.N) st[nb] = *reinterpret_cast<const f32x4*>(st_p + n);
     }
     LOAD_CHUNK(rb, sg.w)
-    STORE_CHUNK()
+    STORE_CHUNK(rb)
     __syncthreads();
     int ck = sg.w;
     for (int t0 = rb; t0 < re; t0 += Q, ++ck) {
@@ -341,54 +416,51 @@ __global__ __launch_bounds__(64 * WPB, 1) void delta_chunk_kernel(const bf16* __
         uint4 tf[2 * FR];
 #pragma unroll
         for (int f = 0; f < 2 * FR; ++f) tf[f] = fr[64 * f];
-        if (more) LOAD_CHUNK(t0 + Q, ck + 1)
+        __builtin_amdgcn_sched_barrier(0);  // loads stay here
+        // products run over independent accumulators: no MFMA waits for the one before it
         f32x4 r[4], o[4];
-        {
-            bf16x8 sh[NB], sl[NB];
 #pragma unroll
-            for (int kb = 0; kb < NB; ++kb) split(st[2 * kb], st[2 * kb + 1], sh[kb], sl[kb]);
+        for (int ib = 0; ib < 4; ++ib) r[ib] = o[ib] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kb = 0; kb < NB; ++kb) {
+            bf16x8 sh, sl, kf[4], qf[4];
 #pragma unroll
             for (int ib = 0; ib < 4; ++ib) {
-                f32x4 ks = {0.f, 0.f, 0.f, 0.f}, qs = {0.f, 0.f, 0.f, 0.f};
-                const int at = (16 * ib + r16) * LK + 4 * g;
+                const int at = row_at<NB>(r16, 32 * kb + 8 * g) + 16 * ib * LK;
+                kf[ib] = *reinterpret_cast<const bf16x8*>(sK + at);
+                qf[ib] = *reinterpret_cast<const bf16x8*>(sQ + at);
+            }
+            split(st[2 * kb], st[2 * kb + 1], sh, sl);
 #pragma unroll
-                for (int kb = 0; kb < NB; ++kb) {
-                    const bf16x8 kf = pair4(sK + at + 32 * kb), qf = pair4(sQ + at + 32 * kb);
-                    ks = mma(kf, sh[kb], ks);
-                    qs = mma(qf, sh[kb], qs);
-                    ks = mma(kf, sl[kb], ks);
-                    qs = mma(qf, sl[kb], qs);
-                }
-                const f32x4 ek = *reinterpret_cast<const f32x4*>(s_vec + 16 * ib + 4 * g);
-                const f32x4 eq = *reinterpret_cast<const f32x4*>(s_vec + 64 + 16 * ib + 4 * g);
-                const s4 vt = tr4(sV + (16 * ib + 4 * g + q4) * LV + 16 * w + p4);
+            for (int ib = 0; ib < 4; ++ib) {
+                r[ib] = mma(kf[ib], sh, r[ib]);
+                o[ib] = mma(qf[ib], sh, o[ib]);
+            }
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    r[ib][e] = __uint_as_float((uint32_t)(uint16_t)vt[e] << 16) - ek[e] * ks[e];
-                    o[ib][e] = eq[e] * qs[e];
-                }
+            for (int ib = 0; ib < 4; ++ib) {
+                r[ib] = mma(kf[ib], sl, r[ib]);
+                o[ib] = mma(qf[ib], sl, o[ib]);
+            }
+        }
+#pragma unroll
+        for (int ib = 0; ib < 4; ++ib) {
+            const f32x4 ek = *reinterpret_cast<const f32x4*>(s_vec + 16 * ib + 4 * g);
+            const f32x4 eq = *reinterpret_cast<const f32x4*>(s_vec + 64 + 16 * ib + 4 * g);
+            const s4 vt = tr4(sV + (16 * ib + 4 * g + q4) * LV + 16 * w + p4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                r[ib][e] = __uint_as_float((uint32_t)(uint16_t)vt[e] << 16) - ek[e] * r[ib][e];
+                o[ib][e] *= eq[e];
             }
         }
         f32x4 u[4];
-        {
-            bf16x8 rh[2], rl[2];
-            split(r[0], r[1], rh[0], rl[0]);
-            split(r[2], r[3], rh[1], rl[1]);
 #pragma unroll
-            for (int ib = 0; ib < 4; ++ib) {
-                u[ib] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int jp = 0; jp <= ib / 2; ++jp) {
-                    const bf16x8 th = __builtin_bit_cast(bf16x8, tf[frag_of(ib, jp)]);
-                    const bf16x8 tl = __builtin_bit_cast(bf16x8, tf[FR + frag_of(ib, jp)]);
-                    u[ib] = mma(th, rh[jp], u[ib]);
-                    u[ib] = mma(th, rl[jp], u[ib]);
-                    u[ib] = mma(tl, rh[jp], u[ib]);
-                }
-            }
-        }
+        for (int ib = 0; ib < 4; ++ib) u[ib] = f32x4{0.f, 0.f, 0.f, 0.f};
+        lower(u, tf, r);
 #pragma unroll
         for (int f = 0; f < 2 * FR; ++f) tf[f] = fr[64 * (2 * FR + f)];  // M
+        LOAD_CHUNK(more ? t0 + Q : t0, more ? ck + 1 : ck)
+        __builtin_amdgcn_sched_barrier(0);  // loads stay here
         {  // state
             const float dec = s_vec[192];
             bf16x8 wh[2], wl[2];
@@ -399,54 +471,227 @@ __global__ __launch_bounds__(64 * WPB, 1) void delta_chunk_kernel(const bf16* __
                 split(u[2 * jp] * w0, u[2 * jp + 1] * w1, wh[jp], wl[jp]);
             }
 #pragma unroll
-            for (int nb = 0; nb < NT; ++nb) {
-                st[nb] *= dec;
+            for (int nb = 0; nb < NT; ++nb) st[nb] *= dec;
+#pragma unroll
+            for (int n4 = 0; n4 < NT; n4 += GN) {
 #pragma unroll
                 for (int jp = 0; jp < 2; ++jp) {
-                    const bf16* kr = sK + (32 * jp + 4 * g + q4) * LK + 16 * nb + p4;
-                    const bf16x8 kt = join(tr4(kr), tr4(kr + 16 * LK));
-                    st[nb] = mma(kt, wh[jp], st[nb]);
-                    st[nb] = mma(kt, wl[jp], st[nb]);
-                }
-            }
-        }
-        {
-            bf16x8 uh[2], ul[2];
-            split(u[0], u[1], uh[0], ul[0]);
-            split(u[2], u[3], uh[1], ul[1]);
+                    bf16x8 kt[GN];
 #pragma unroll
-            for (int ib = 0; ib < 4; ++ib) {
-#pragma unroll
-                for (int jp = 0; jp <= ib / 2; ++jp) {
-                    const bf16x8 mh = __builtin_bit_cast(bf16x8, tf[frag_of(ib, jp)]);
-                    const bf16x8 ml = __builtin_bit_cast(bf16x8, tf[FR + frag_of(ib, jp)]);
-                    o[ib] = mma(mh, uh[jp], o[ib]);
-                    o[ib] = mma(mh, ul[jp], o[ib]);
-                    o[ib] = mma(ml, uh[jp], o[ib]);
-                }
-                if (p < a.P) {
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        const int t = t0 + 16 * ib + 4 * g + e;
-                        if (t < re) y[(size_t)(t - y0) * inner + head * a.P + p] = o[ib][e];
+                    for (int i = 0; i < GN; ++i) {
+                        const bf16* kr = sK + row_at<NB>(4 * g + q4, tile_row(n4 + i, r16 & 3)) + 32 * jp * LK;
+                        kt[i] = join(tr4(kr), tr4(kr + 16 * LK));
                     }
+#pragma unroll
+                    for (int i = 0; i < GN; ++i) st[n4 + i] = mma(kt[i], wh[jp], st[n4 + i]);
+#pragma unroll
+                    for (int i = 0; i < GN; ++i) st[n4 + i] = mma(kt[i], wl[jp], st[n4 + i]);
                 }
             }
         }
+        lower(o, tf, u);
+        STORE_ROWS(o)
         if (more) {
             __syncthreads();  // every wave is done with this chunk's LDS images
-            STORE_CHUNK()
+            STORE_CHUNK(t0 + Q)
             __syncthreads();
         }
     }
-#undef LOAD_CHUNK
-#undef STORE_CHUNK
     if (p < a.P) {
 #pragma unroll
         for (int nb = 0; nb < NT; ++nb)
-            if (16 * nb + 4 * g < a.N) *reinterpret_cast<f32x4*>(st_p + 16 * nb) = st[nb];
+            if (tile_row(nb, g) < a.N) *reinterpret_cast<f32x4*>(st_p + tile_row(nb, g)) = st[nb];
     }
 }
+
+// The same with two waves per 16 value columns, for grids that leave SIMDs idle: one carries the state (its chain is what a
+// chunk takes), the other turns the state at the chunk's start and U into output rows beside it.  Both reach it as finished
+// operands through LDS.
+template <int NB, int WPB>
+__global__ __launch_bounds__(128 * WPB, 1) void delta_chunk_pair_kernel(const bf16* __restrict__ x, DeltaArgs a,
+                                                                        const int4* __restrict__ segs,
+                                                                        const int* __restrict__ slots,
+                                                                        const int* __restrict__ pos0,
+                                                                        const uint4* __restrict__ frags,
+                                                                        const float* __restrict__ vec,
+                                                                        float* __restrict__ state, float* __restrict__ y,
+                                                                        int y0) {
+    constexpr int NTH = 128 * WPB, NN = 32 * NB, LK = row_stride<NB>(), LV = 16 * WPB + 16, NT = 2 * NB, GN = NT < 4 ? NT : 4;
+    constexpr int KIT = (Q * 4 * NB + NTH - 1) / NTH, VR = 1;
+    constexpr int VIT = NTH < 256 ? 256 / NTH : 1;
+    __shared__ __attribute__((aligned(16))) bf16 sK[Q * LK];
+    __shared__ __attribute__((aligned(16))) bf16 sQ[Q * LK];
+    __shared__ __attribute__((aligned(16))) bf16 sV[Q * LV];
+    __shared__ __attribute__((aligned(16))) float s_vec[256];
+    __shared__ bf16x8 sS[WPB][2 * NB][64];  // state operands, hi and lo
+    __shared__ bf16x8 sU[WPB][4][64];       // U operands, hi and lo
+    const int head = blockIdx.x, pb = 16 * WPB * blockIdx.y;
+    const int4 sg = segs[blockIdx.z];
+    const int rb = sg.y, re = sg.z;
+    const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, g = lane >> 4, q4 = r16 >> 2, p4 = 4 * (r16 & 3);
+    const int wv = __builtin_amdgcn_readfirstlane(tid >> 6), w = wv % WPB;
+    const int kh = head / (a.heads / a.kv_heads), inner = a.heads * a.P;
+    const bf16* qcol = x + kh * a.N;
+    const bf16* kcol = qcol + a.xk;
+    const bf16* vcol = x + a.xv + head * a.P + pb;
+    const int p = pb + 16 * w + r16;  // this lane's value column
+    u32x4 kreg[KIT], qreg[KIT], vreg[VR];
+    float vecr[VIT];
+    const uint4* fr = frags + ((size_t)sg.w * a.heads + head) * FRAGS + lane;  // this chunk's T and M
+    const size_t fr_step = (size_t)a.heads * FRAGS;
+    uint4 lf[2 * FR];
+    int ck = sg.w;
+    if (wv < WPB) {
+        float* st_p = state + ((size_t)slots[sg.x] * a.heads + head) * a.P * a.N4 + (size_t)p * a.N4;
+        f32x4 st[NT];
+        const bool cont = pos0[sg.x] > 0;
+#pragma unroll
+        for (int nb = 0; nb < NT; ++nb) {
+            st[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const int n = tile_row(nb, g);
+            if (cont && p < a.P && n < a.N) st[nb] = *reinterpret_cast<const f32x4*>(st_p + n);
+        }
+        bf16x8 sh[NB], sl[NB];
+#define PUBLISH()                                                         \
+    _Pragma("unroll") for (int kb = 0; kb < NB; ++kb) {                   \
+        split(st[2 * kb], st[2 * kb + 1], sh[kb], sl[kb]);                \
+        sS[w][kb][lane] = sh[kb];                                         \
+        sS[w][NB + kb][lane] = sl[kb];                                    \
+    }
+#pragma unroll
+        for (int f = 0; f < 2 * FR; ++f) lf[f] = fr[64 * f];
+        LOAD_CHUNK(rb, ck)
+        STORE_CHUNK(rb)
+        PUBLISH()
+        __syncthreads();
+        for (int t0 = rb; t0 < re; t0 += Q) {
+            const bool more = t0 + Q < re;
+            LOAD_CHUNK(more ? t0 + Q : t0, more ? ck + 1 : ck)
+            __builtin_amdgcn_sched_barrier(0);  // loads stay here
+            f32x4 r[4], u[4];
+#pragma unroll
+            for (int ib = 0; ib < 4; ++ib) r[ib] = u[ib] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kb = 0; kb < NB; ++kb) {
+                bf16x8 kf[4];
+#pragma unroll
+                for (int ib = 0; ib < 4; ++ib)
+                    kf[ib] = *reinterpret_cast<const bf16x8*>(sK + row_at<NB>(r16, 32 * kb + 8 * g) + 16 * ib * LK);
+#pragma unroll
+                for (int ib = 0; ib < 4; ++ib) r[ib] = mma(kf[ib], sh[kb], r[ib]);
+#pragma unroll
+                for (int ib = 0; ib < 4; ++ib) r[ib] = mma(kf[ib], sl[kb], r[ib]);
+            }
+#pragma unroll
+            for (int ib = 0; ib < 4; ++ib) {
+                const f32x4 ek = *reinterpret_cast<const f32x4*>(s_vec + 16 * ib + 4 * g);
+                const s4 vt = tr4(sV + (16 * ib + 4 * g + q4) * LV + 16 * w + p4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    r[ib][e] = __uint_as_float((uint32_t)(uint16_t)vt[e] << 16) - ek[e] * r[ib][e];
+            }
+            lower(u, lf, r);
+            {
+                bf16x8 h, l;
+#pragma unroll
+                for (int jp = 0; jp < 2; ++jp) {
+                    split(u[2 * jp], u[2 * jp + 1], h, l);
+                    sU[w][jp][lane] = h;
+                    sU[w][2 + jp][lane] = l;
+                }
+            }
+            __syncthreads();  // U is in LDS; the output waves have read the state
+            if (more) fr += fr_step;
+#pragma unroll
+            for (int f = 0; f < 2 * FR; ++f) lf[f] = fr[64 * f];
+            const float dec = s_vec[192];
+            bf16x8 wh[2], wl[2];
+#pragma unroll
+            for (int jp = 0; jp < 2; ++jp) {
+                const f32x4 w0 = *reinterpret_cast<const f32x4*>(s_vec + 128 + 32 * jp + 4 * g);
+                const f32x4 w1 = *reinterpret_cast<const f32x4*>(s_vec + 128 + 32 * jp + 16 + 4 * g);
+                split(u[2 * jp] * w0, u[2 * jp + 1] * w1, wh[jp], wl[jp]);
+            }
+#pragma unroll
+            for (int nb = 0; nb < NT; ++nb) st[nb] *= dec;
+#pragma unroll
+            for (int n4 = 0; n4 < NT; n4 += GN)
+#pragma unroll
+                for (int jp = 0; jp < 2; ++jp) {
+                    bf16x8 kt[GN];
+#pragma unroll
+                    for (int i = 0; i < GN; ++i) {
+                        const bf16* kr = sK + row_at<NB>(4 * g + q4, tile_row(n4 + i, r16 & 3)) + 32 * jp * LK;
+                        kt[i] = join(tr4(kr), tr4(kr + 16 * LK));
+                    }
+#pragma unroll
+                    for (int i = 0; i < GN; ++i) st[n4 + i] = mma(kt[i], wh[jp], st[n4 + i]);
+#pragma unroll
+                    for (int i = 0; i < GN; ++i) st[n4 + i] = mma(kt[i], wl[jp], st[n4 + i]);
+                }
+            if (more) {
+                __syncthreads();  // every wave is done with this chunk's LDS images
+                STORE_CHUNK(t0 + Q)
+                PUBLISH()
+                __syncthreads();
+                ++ck;
+            }
+        }
+#undef PUBLISH
+        if (p < a.P) {
+#pragma unroll
+            for (int nb = 0; nb < NT; ++nb)
+                if (tile_row(nb, g) < a.N) *reinterpret_cast<f32x4*>(st_p + tile_row(nb, g)) = st[nb];
+        }
+        return;
+    }
+    fr += 64 * 2 * FR;
+#pragma unroll
+    for (int f = 0; f < 2 * FR; ++f) lf[f] = fr[64 * f];
+    LOAD_CHUNK(rb, ck)
+    STORE_CHUNK(rb)
+    __syncthreads();
+    for (int t0 = rb; t0 < re; t0 += Q) {
+        const bool more = t0 + Q < re;
+        LOAD_CHUNK(more ? t0 + Q : t0, more ? ck + 1 : ck)
+        __builtin_amdgcn_sched_barrier(0);  // loads stay here
+        f32x4 o[4];
+#pragma unroll
+        for (int ib = 0; ib < 4; ++ib) o[ib] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kb = 0; kb < NB; ++kb) {
+            const bf16x8 sh = sS[w][kb][lane], sl = sS[w][NB + kb][lane];
+            bf16x8 qf[4];
+#pragma unroll
+            for (int ib = 0; ib < 4; ++ib)
+                qf[ib] = *reinterpret_cast<const bf16x8*>(sQ + row_at<NB>(r16, 32 * kb + 8 * g) + 16 * ib * LK);
+#pragma unroll
+            for (int ib = 0; ib < 4; ++ib) o[ib] = mma(qf[ib], sh, o[ib]);
+#pragma unroll
+            for (int ib = 0; ib < 4; ++ib) o[ib] = mma(qf[ib], sl, o[ib]);
+        }
+#pragma unroll
+        for (int ib = 0; ib < 4; ++ib) o[ib] *= *reinterpret_cast<const f32x4*>(s_vec + 64 + 16 * ib + 4 * g);
+        __syncthreads();  // U is in LDS; the state has been read
+        {
+            const bf16x8 hi[2] = {sU[w][0][lane], sU[w][1][lane]}, lo[2] = {sU[w][2][lane], sU[w][3][lane]};
+            lower(o, lf, hi, lo);
+        }
+        if (more) fr += fr_step;
+#pragma unroll
+        for (int f = 0; f < 2 * FR; ++f) lf[f] = fr[64 * f];
+        STORE_ROWS(o)
+        if (more) {
+            __syncthreads();  // every wave is done with this chunk's LDS images
+            STORE_CHUNK(t0 + Q)
+            __syncthreads();
+            ++ck;
+        }
+    }
+}
+#undef LOAD_CHUNK
+#undef STORE_CHUNK
+#undef STORE_ROWS
 
 // 16-byte pieces and floats of workspace per (chunk, head)
 MRSUM_API int mrsum_delta_chunk_pieces() { return FRAGS; }
@@ -454,20 +699,24 @@ MRSUM_API int mrsum_delta_chunk_pieces() { return FRAGS; }
 // Segments of ``segs`` (segment, first row, end row, first chunk); chunks (first row, end row) of at most 64 rows each, in
 // order.  x [T][ldx] bf16; frags [n_chunks][heads][FRAGS] 16-byte pieces, vec [n_chunks][heads][256] fp32: workspace.
 // y: fp32 rows [T - y0][heads * P] from row y0 on.  P % 8 == 0, N % 8 == 0, N <= 256.  wpb: waves of 16 value columns per
-// block (2, 4, or up to N = 128 also 8).
+// block (2, 4, or up to N = 128 also 8); pair: two waves each (2 or 4, N <= 128).
 MRSUM_API int mrsum_delta_chunk(const void* x, int ldx, int xk, int xv, const void* u, int S, int ld, int T, int b_at,
                                 int a_at, const float* dt_bias, const float* a_neg, float* state, const int* slots,
                                 const int* pos0, const void* segs, int n_segs, const void* chunks, int n_chunks, void* frags,
-                                float* vec, float* y, int y0, int heads, int kv_heads, int P, int N, int wpb, hipStream_t s) {
+                                float* vec, float* y, int y0, int heads, int kv_heads, int P, int N, int wpb, int pair,
+                                hipStream_t s) {
     if (T <= 0 || n_segs <= 0) return 0;
     if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || heads > 65535 || n_segs > 65535 || n_chunks > 65535 ||
         n_chunks < n_segs || P <= 0 || N <= 0 || P % 8 || N % 8 || N > 256 || ldx % 8 || xk % 8 || xv % 8 ||
         xk < kv_heads * N || xv < xk + kv_heads * N || ldx < xv + heads * P || b_at + heads > ld || a_at + heads > ld ||
-        (wpb != 2 && wpb != 4 && (wpb != 8 || N > 128)))
+        (wpb != 2 && wpb != 4 && (wpb != 8 || N > 128)) || (pair && (wpb == 8 || N > 128)))
         return (int)hipErrorInvalidValue;
     const DeltaArgs a{ProjSrc{u, S, (size_t)T * ld, ld}, b_at, a_at, 0, dt_bias, a_neg, nullptr, 0.f,
                       1.f / sqrtf((float)N), ldx, xk, xv, 0, 0, 0, heads, kv_heads, P, N, N};
-    const dim3 g1(kv_heads, n_chunks), g2(ceil_div(P, 16 * wpb), heads, n_segs);
+    const dim3 g1(kv_heads, n_chunks), g2(heads, ceil_div(P, 16 * wpb), n_segs);
+#define DC_P(NB_, W_)                                                                                                     \
+    delta_chunk_pair_kernel<NB_, W_><<<g2, 128 * W_, 0, s>>>((const bf16*)x, a, (const int4*)segs, slots, pos0,              \
+                                                            (const uint4*)frags, vec, state, y, y0)
 #define DC_W(NB_, W_)                                                                                                     \
     delta_chunk_kernel<NB_, W_><<<g2, 64 * W_, 0, s>>>((const bf16*)x, a, (const int4*)segs, slots, pos0, (const uint4*)frags, \
                                                        vec, state, y, y0)
@@ -476,9 +725,11 @@ MRSUM_API int mrsum_delta_chunk(const void* x, int ldx, int xk, int xv, const vo
         delta_prep_kernel<NB_><<<g1, 256, 0, s>>>((const bf16*)x, a, (const int2*)chunks, (uint4*)frags, vec); \
         if constexpr (NB_ < 8) {                                                                             \
             if (wpb == 8) DC_W(NB_, 8);                                                                      \
+            else if (wpb == 4 && pair) DC_P(NB_, 4);                                                              \
+            else if (wpb == 2 && pair) DC_P(NB_, 2);                                                         \
         }                                                                                                    \
-        if (wpb == 4) DC_W(NB_, 4);                                                                          \
-        else if (wpb == 2) DC_W(NB_, 2);                                                                     \
+        if (wpb == 4 && !pair) DC_W(NB_, 4);                                                                 \
+        else if (wpb == 2 && !pair) DC_W(NB_, 2);                                                            \
     }
     if (N <= 32) DC(1)
     else if (N <= 64) DC(2)
@@ -486,5 +737,6 @@ MRSUM_API int mrsum_delta_chunk(const void* x, int ldx, int xk, int xv, const vo
     else DC(8)
 #undef DC
 #undef DC_W
+#undef DC_P
     return (int)hipGetLastError();
 }

@@ -87,7 +87,8 @@ _SIGS = {
                              _vp, _c_int, _c_int, _vp, _c_int, _c_float, _c_int, _vp],
     "mrsum_latent_decode": [_vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _vp, _vp, _vp],
     "mrsum_delta_chunk": [_vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp,
-                          _vp, _c_int, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp],
+                          _vp, _c_int, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                          _vp],
     "mrsum_delta_chunk_pieces": [],
     "mrsum_delta_step": [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp,
                          _vp, _c_float, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int,
@@ -1968,12 +1969,14 @@ def delta_chunks(lens, first: int):
     return segs, chunks
 
 
-def delta_waves(vdim: int, dim: int, pairs: int) -> int:
-    """Waves of 16 value columns per workgroup: as many as leave no CU without a workgroup."""
-    for w in (8, 4) if dim <= 128 else (4,):
-        if 16 * (w // 2) < vdim and pairs * -(-vdim // (16 * w)) >= N_CU:
-            return w
-    return 2
+def delta_waves(vdim: int, dim: int, pairs: int):
+    """(blocks of 16 value columns per workgroup, two waves per block or one) of ``pairs`` (segment, head) pairs: as many
+    blocks as leave no CU without a workgroup; below that, pairs of waves."""
+    if dim > 128:
+        return (4, 0) if vdim > 32 and pairs * -(-vdim // 64) >= N_CU else (2, 0)
+    if vdim > 64 and pairs * -(-vdim // 128) >= N_CU:
+        return 8, 0
+    return (4 if vdim > 32 and pairs * -(-vdim // 64) >= N_CU else 2), 1
 
 
 def delta_mix(x, u, m, a_neg, dt_bias, norm, eps: float, state, segs, a) -> None:
@@ -2009,7 +2012,7 @@ def delta_mix(x, u, m, a_neg, dt_bias, norm, eps: float, state, segs, a) -> None
         y = torch.empty(T - y0, H * P, dtype=torch.float32, device=u.device)
         _check(_fn("mrsum_delta_chunk")(_p(x), x.shape[1], m.xk, m.xv, ptr, S, ld, T, m.b, m.a, _p(dt_bias), _p(a_neg),
                                         _p(state), _p(segs.slots), _p(segs.pos0), _p(runs), runs.shape[0], _p(chunks), nc,
-                                        _p(frags), _p(vec), _p(y), y0, H, G, P, N, delta_waves(P, N, H * runs.shape[0]),
+                                        _p(frags), _p(vec), _p(y), y0, H, G, P, N, *delta_waves(P, N, H * runs.shape[0]),
                                         _stream()), "delta_chunk")
         rows = a[y0:]
         _check(_fn("mrsum_gated_norm")(_p(y), ptr + y0 * ld * (4 if S else 2), S, ld, T - y0, m.g, _p(norm), H * P, H, eps,

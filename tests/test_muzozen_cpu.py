@@ -231,8 +231,9 @@ def test_work_lists_cover_every_row():
         items = block_items(lens, 256).tolist()
         assert sorted(map(tuple, items)) == sorted((i, q) for i, n in enumerate(lens) for q in range(0, n, 256))
         assert [q for _, q in items] == sorted((q for _, q in items), reverse=True)
-    for P, N, pairs in ((128, 128, 256), (128, 128, 32), (64, 128, 512), (16, 32, 4), (136, 200, 999)):
-        assert delta_waves(P, N, pairs) in ((2, 4, 8) if N <= 128 else (2, 4))
+    for P, N, pairs, want in ((128, 128, 256, (8, 0)), (128, 128, 128, (4, 1)), (128, 128, 32, (2, 1)), (16, 32, 4, (2, 1)),
+                              (48, 128, 512, (4, 1)), (136, 200, 999, (4, 0)), (24, 256, 999, (2, 0))):
+        assert delta_waves(P, N, pairs) == want
 
 
 def test_portion_context_places_every_page():

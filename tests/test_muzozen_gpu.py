@@ -186,6 +186,12 @@ def test_latent_attention_finds_the_key_that_stands_out(H, dim, rd, vdim, rank, 
                 out = blank(len(last))
                 ops.latent_out_parts(parts, m, m.w.w_uv, out, 8)
                 same(out, last, "decode %d" % splits)
+            many = ix.repeat(26)  # enough rows that a merging block takes several
+            parts = ops.latent_decode(qa[many].contiguous(), cache, bt.repeat(26, 1), pos[many].contiguous(), H, m.rank8, page,
+                                      spec.scale, None)
+            out = blank(len(many))
+            ops.latent_out_parts(parts, m, m.w.w_uv, out, 8)
+            same(out, last * 26, "decode of many rows")
         if not m.flash or (qsrc.dim() == 3 and T > 64 and H > 8):
             continue
         for nd in ((0, 3) if H < 9 else (0,)):
@@ -223,12 +229,13 @@ DELTA = [(4, 2, 128, 128), (3, 3, 24, 40), (2, 1, 64, 136), (6, 2, 32, 16), (2, 
 
 @pytest.mark.parametrize("H,G,dim,vdim", DELTA)
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_delta_rule(H, G, dim, vdim, dtype):
+def test_delta_rule(H, G, dim, vdim, dtype, monkeypatch):
     """Decoded rows, short and long portions, fresh and continued slots holding garbage or carried state, keys that repeat
     (so that corrections chain through a chunk), decays from almost none to total, output norm and gate."""
     from llm_map_reduce_summarizer_amd import ops
     from llm_map_reduce_summarizer_amd.engine import mixers
     from llm_map_reduce_summarizer_amd.engine.config import DeltaSpec
+    from llm_map_reduce_summarizer_amd.ops import hip
     m = mixers.DeltaMixer(DeltaSpec(H, G, dim, vdim, 2), torch.device(DEV), dtype)
     cols = [0]
 
@@ -253,9 +260,13 @@ def test_delta_rule(H, G, dim, vdim, dtype):
     slots, pos0 = [3, 1, 5, 2, 6, 4], [9, 0, 7, 64, 0, 1000]
     init = rnd(len(lens), H, dim, vdim, seed=6, std=0.5)
     N4 = dim + (-dim) % 4
-    for src, dt_, vals in forms(u):
-        if dt_ != dtype:
-            continue
+    sets = [s for s in forms(u) if s[1] == dtype]
+    if dtype == BF and hip.delta_chunk_ok(vdim, dim):  # every form of the chunked kernel
+        waves = [(8, 0), (4, 0), (4, 1), (2, 0), (2, 1)] if dim <= 128 else [(4, 0), (2, 0)]
+        sets = [s + (w,) for s, w in zip(sets * len(waves), waves + waves[::-1])]
+    for src, dt_, vals, *w in sets:
+        if w:
+            monkeypatch.setattr(hip, "delta_waves", lambda *_, w=w[0]: w)
         state = torch.full((8, H, vdim, N4), 1e4, device=DEV)
         state[..., dim:] = 0
         for i, s in enumerate(slots):
@@ -312,6 +323,16 @@ def test_long_prompt_then_long_decoding(dtype, tmp_path):
     eng = M.engine("wide", tmp_path, DEV, dtype, max_model_len=1024)
     ids = M.tokens("wide", 700)
     M.check(M.feed(eng, "a", ids, [600] + [1] * 100), M.expected("wide", ids), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_prompt_of_more_than_a_thousand_rows(dtype, tmp_path):
+    """Row counts from which on the preparation and norm kernels change their form, in one portion and in three."""
+    eng = M.engine("mixed", tmp_path, DEV, dtype, max_model_len=1280)
+    ids = M.tokens("mixed", 1130)
+    want = M.expected("mixed", ids)
+    M.check(M.feed(eng, "a", ids, [1100] + [1] * 30), want, dtype, "one portion")
+    M.check(M.feed(eng, "b", ids, [70, 1030, 2] + [1] * 28), want, dtype, "portions")
 
 
 @pytest.mark.parametrize("name", ["mixed", "wide"])
