@@ -11,6 +11,13 @@
 #include "common.h"
 #include "delta.h"
 
+__device__ __forceinline__ float4 in4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+__device__ __forceinline__ float4 in4(const bf16* p) {
+    const uint2 v = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+                       __uint_as_float(v.y & 0xffff0000u));
+}
+
 // One block per (head, segment): LPR lanes hold a state row (one value column) as NV float4 each, R rows per lane group.
 template <bool PARTS, typename T, int NT, int LPR, int NV, int R>
 __global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x, DeltaArgs a, SegArgs sg, int seg0,
@@ -33,6 +40,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x,
             S[i][v] = make_float4(0.f, 0.f, 0.f, 0.f);
             if (cont && p < a.P && n < a.N4) S[i][v] = *reinterpret_cast<const float4*>(st + (size_t)p * a.N4 + n);
         }
+    const bool whole = a.N % 4 == 0 && a.ldx % 4 == 0 && a.xk % 4 == 0;
     const float an = a.a_neg[head], db = a.dt_bias[head];
     for (int t = b; t < e; ++t) {
         const T* row = x + (size_t)t * a.ldx;
@@ -43,15 +51,27 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x,
         float qq = 0.f, kk = 0.f, kq = 0.f;
 #pragma unroll
         for (int v = 0; v < NV; ++v)
+        {
+            const int n0 = 4 * (l + LPR * v);
+            if (whole) {  // four neighbouring columns at once
+                const float4 qv = in4(row + kh * a.N + min(n0, a.N - 4)), kv = in4(row + a.xk + kh * a.N + min(n0, a.N - 4));
+                const float on = n0 < a.N ? 1.f : 0.f;
+                q[v][0] = on * qv.x; q[v][1] = on * qv.y; q[v][2] = on * qv.z; q[v][3] = on * qv.w;
+                k[v][0] = on * kv.x; k[v][1] = on * kv.y; k[v][2] = on * kv.z; k[v][3] = on * kv.w;
+            } else {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    q[v][j] = n0 + j < a.N ? (float)row[kh * a.N + n0 + j] : 0.f;
+                    k[v][j] = n0 + j < a.N ? (float)row[a.xk + kh * a.N + n0 + j] : 0.f;
+                }
+            }
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                const int n = 4 * (l + LPR * v) + j;
-                q[v][j] = n < a.N ? (float)row[kh * a.N + n] : 0.f;
-                k[v][j] = n < a.N ? (float)row[a.xk + kh * a.N + n] : 0.f;
                 qq += q[v][j] * q[v][j];
                 kk += k[v][j] * k[v][j];
                 kq += k[v][j] * q[v][j];
             }
+        }
         const float beta = logistic(proj_at<PARTS>(a.u, t, a.b_at + head));
         const float g = expf(an * softplus(proj_at<PARTS>(a.u, t, a.a_at + head) + db));
 #pragma unroll
@@ -140,6 +160,7 @@ static int launch_delta_step(const void* x, const DeltaArgs& a, const SegArgs& s
     }
     if (q <= 8) DS_R(256, 8, 1)
     else if (q <= 16) DS_R(256, 16, 1)
+    else if (q <= 32 && a.P > 64 && a.P <= 128 && a.heads * nseg <= 256) DS(1024, 32, 1, 4);  // one block per CU
     else if (q <= 32) DS_R(512, 32, 1)
     else if (q <= 64) DS_R(512, 64, 1)
     else return (int)hipErrorInvalidValue;
