@@ -20,7 +20,7 @@ __device__ __forceinline__ float4 in4(const bf16* p) {
 
 // One block per (head, segment): LPR lanes hold a state row (one value column) as NV float4 each, R rows per lane group.
 template <bool PARTS, typename T, int NT, int LPR, int NV, int R>
-__global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x, DeltaArgs a, SegArgs sg, int seg0,
+__global__ __launch_bounds__(NT, R <= 8 ? 4 : 1) void delta_step_kernel(const T* __restrict__ x, DeltaArgs a, SegArgs sg, int seg0,
                                                         float* __restrict__ state, T* __restrict__ out) {
     constexpr int RP = NT / LPR;
     __shared__ float s_o[RP * R];
@@ -81,7 +81,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const T* __restrict__ x,
             kq += __shfl_xor(kq, o, 64);
         }
         const float rk = 1.f / sqrtf(kk + 1e-6f), rq = a.q_scale / sqrtf(qq + 1e-6f);
-        constexpr int GR = R < 8 ? R : 8;  // rows reduced together
+        constexpr int GR = R < 4 ? R : 4;  // rows reduced together
 #pragma unroll
         for (int i0 = 0; i0 < R; i0 += GR) {
             float sk[GR], sq[GR], vv[GR];
