@@ -352,7 +352,7 @@ PRESETS = {
     "muzozen-8b": _muzozen("muzozen-8b", 128256, 4096, "LSDD" * 8,
                            latent=LatentSpec(32, 128, 128, 1536, 512,
                                              RotarySpec(64, 500000.0, YarnSpec(8.0, 8192, 32.0, 1.0)), 192 ** -0.5),
-                           delta=DeltaSpec(32, 16, 128, 128, 4), ff=18432, bigram=BigramSpec(65536, 31, 7),
+                           delta=DeltaSpec(32, 16, 128, 128, 4), ff=18432, bigram=BigramSpec(65536, 8191, 127),
                            embed_scale=8.0),
     "tiny-muzozen": _muzozen("tiny-muzozen", 128256, 192, "LdSD",
                              latent=LatentSpec(4, 48, 32, 72, 96, RotarySpec(24, 10000.0, YarnSpec(2.0, 512, 16.0, 1.0)),

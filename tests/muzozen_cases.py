@@ -56,7 +56,7 @@ CONFIGS = {
     "wide": config(130, 256, [
         latent(8, 128, 128, 192, 512, rot(64, base=500000.0), ff=192),
         delta(4, 2, 128, 128, 4, ff=256),
-        latent(8, 128, 128, 192, 512, rot(64, base=500000.0), kv_from=0)], buckets=509),
+        latent(8, 128, 128, 192, 512, rot(64, base=500000.0), kv_from=0)], buckets=503),
     # more heads than a decode workgroup takes; medium latents; wide delta values
     "many_heads": config(65, 96, [
         latent(40, 64, 48, 64, 200, rot(32), ff=64),
